@@ -10,6 +10,7 @@ import os
 
 HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(HERE, "libvui_amd.so")
+LM_LIB_PATH = os.path.join(HERE, "libvui_lm.so")
 
 VUI_MAX_LAYERS = 64
 VUI_MAX_RQ_LAYERS = 16
@@ -65,6 +66,34 @@ class CodecConfigC(C.Structure):
         ("n_rates", C.c_int32), ("rates", C.c_int32 * 8)]
 
 
+class LmConfigC(C.Structure):
+    """vui_lm_config (include/vui_lm.h)."""
+    _fields_ = [(n, C.c_int32) for n in ("dtype", "width", "vocab", "n_layers", "max_seqlen", "n_slots", "max_rows")] + [
+        ("norm_eps", C.c_float)]
+
+
+class LmLayerC(C.Structure):
+    """vui_lm_layer."""
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "kv_from", "heads", "dim", "rot_dim", "rot_pairs", "vdim", "kv_rank")] + [
+        ("scale", C.c_float), ("rnn_width", C.c_int32), ("ff", C.c_int32), ("limit", C.c_float)] + [(n, C.c_void_p) for n in (
+            "norm", "w_in", "w_out", "w_uk_t", "w_uk", "w_uv", "latent_norm", "rope", "bias_z", "bias_x", "c_cache", "kr_cache", "state")]
+
+
+class LmDimsC(C.Structure):
+    """vui_lm_dims."""
+    _fields_ = [(n, C.c_int32) for n in (
+        "w16", "w64", "s64", "dim16", "dim64", "rot16", "rot32", "rank16", "rank64", "vdim16", "heads16", "gru16",
+        "mix_rows", "in_rows", "ff_pad", "ff_off", "out_k", "out_rows")]
+
+
+class LmWeightsC(C.Structure):
+    """vui_lm_weights."""
+    _fields_ = [("embed", C.c_void_p), ("head", C.c_void_p), ("final_norm", C.c_void_p)]
+
+
+LM_LATENT_ATTENTION, LM_MINGRU = 0, 1
+
+
 # name -> (restype, argtypes); every symbol include/*.h declares
 _P, _I, _L, _F = C.c_void_p, C.c_int, C.c_int64, C.c_float
 SIGNATURES = {
@@ -109,35 +138,54 @@ SIGNATURES = {
     "vui_attn_scratch_bytes": (_L, [_I, _I, _I, _I]),
     "vui_decode_attn": (_I, [_I, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P]),
     "vui_decode_attn_noalloc": (_I, [_I, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P]),
+    "vui_lm_layer_dims": (_I, [C.POINTER(LmConfigC), C.POINTER(LmLayerC), C.POINTER(LmDimsC)]),
+    "vui_lm_workspace_bytes": (_L, [C.POINTER(LmConfigC), C.POINTER(LmLayerC)]),
+    "vui_lm_create": (_I, [C.POINTER(LmConfigC), C.POINTER(LmLayerC), C.POINTER(LmWeightsC), _P, _L, C.POINTER(_P)]),
+    "vui_lm_destroy": (None, [_P]),
+    "vui_lm_decode": (_I, [_P, _P, _P, _P, _P, _I, _P, _P]),
+    "vui_lm_prefill": (_I, [_P, _P, _I, _I, _I, _P, _P, _I, _P, _P]),
+    "vui_lm_debug_layers": (_I, [_P, _P]),
+    "vui_lm_expand_from": (_I, [_P, _I]),
+    "vui_sample_tokens": (_I, [_P, _I, _P, _P, _P, _F, _I, C.POINTER(SampleParamsC), _P, _I, _P]),
     "vui_sample_logits": (_I, [_P, _P, _I, C.POINTER(SampleParamsC), _I, _P, _I, _P]),
 }
 
 _lib = None
+_lib_part = False
 
 
-def load() -> C.CDLL:
-    """Loads the shared library (once) and types its entry points."""
-    global _lib
+def load(lm_only: bool = False) -> C.CDLL:
+    """Loads the shared library (once) and types its entry points.  lm_only: the caller needs the token language
+    models, the sampler and the graph helpers only; where the whole library has not been built, the part of it that
+    `vui_amd.build.build_lm` compiles will do."""
+    global _lib, _lib_part
     if _lib is not None:
+        if _lib_part and not lm_only:
+            raise RuntimeError("only the token language models' part of the library is built: `python -m vui_amd.build`")
         return _lib
-    if not os.path.exists(LIB_PATH):
+    path, part = LIB_PATH, False
+    if lm_only and not os.path.exists(path):
+        path, part = LM_LIB_PATH, True
+    if not os.path.exists(path):
         raise RuntimeError(
             f"{LIB_PATH} is missing: build it with `python -m vui_amd.build` (there is no fallback path)")
     # one HIP runtime per process: PyTorch brings its own copy, so it is loaded first and the library binds
     # to that one (loaded the other way round, kernels launched from here find no device)
     import torch  # noqa: F401
 
-    lib = C.CDLL(LIB_PATH)
+    lib = C.CDLL(path)
     for name, (res, args) in SIGNATURES.items():
+        if part and not hasattr(lib, name):
+            continue
         fn = getattr(lib, name)  # AttributeError if the library does not export it
         fn.restype = res
         fn.argtypes = args
-    _lib = lib
+    _lib, _lib_part = lib, part
     return lib
 
 
 def last_error() -> str:
-    return load().vui_last_error().decode("utf-8", "replace")
+    return load(lm_only=True).vui_last_error().decode("utf-8", "replace")
 
 
 def check(rc: int, what: str) -> None:

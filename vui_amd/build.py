@@ -9,7 +9,11 @@ from concurrent.futures import ThreadPoolExecutor
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libvui_amd.so")
-SOURCES = ["gemv.hip", "gemm16.hip", "attn.hip", "misc.hip", "frame.hip", "rqbatch.hip", "bbatch.hip", "prefill.hip", "codec.hip", "api.hip"]
+# the token language models alone: their kernels, the sampler, the graph helpers
+LM_LIB = os.path.join(HERE, "libvui_lm.so")
+LM_SOURCES = ["runtime.hip", "misc.hip", "lm_gemm.hip", "latent.hip", "scan.hip", "lm.hip"]
+SOURCES = ["gemv.hip", "gemm16.hip", "attn.hip", "misc.hip", "frame.hip", "rqbatch.hip", "bbatch.hip", "prefill.hip", "codec.hip", "api.hip",
+           "runtime.hip", "lm_gemm.hip", "latent.hip", "scan.hip", "lm.hip"]
 FLAGS = [
     "-O3", "--offload-arch=gfx950", "-fPIC", "-std=c++17", "-Wall", "-Wno-unused-function",
     # packed-fp32 instructions are kept out of every code object of this library
@@ -24,8 +28,7 @@ def _hipcc() -> str:
     return "hipcc"
 
 
-def build(verbose: bool = True) -> str:
-    """Compiles every translation unit and links the shared library.  Always recompiles."""
+def _build(lib: str, sources: "list[str]", verbose: bool) -> str:
     hipcc = _hipcc()
     extra = os.environ.get("VUI_EXTRA_HIPCC_FLAGS", "").split()
     objdir = os.path.join(CSRC, "build")
@@ -43,15 +46,27 @@ def build(verbose: bool = True) -> str:
                 print("\n".join(lines), file=sys.stderr)
         return obj
 
-    with ThreadPoolExecutor(max_workers=min(8, len(SOURCES))) as ex:
-        objs = list(ex.map(one, SOURCES))
-    cmd = [hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB, *objs]
+    with ThreadPoolExecutor(max_workers=min(8, len(sources))) as ex:
+        objs = list(ex.map(one, sources))
+    tmp = lib + ".tmp"
+    cmd = [hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", tmp, *objs]
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError(f"link failed:\n{r.stdout}\n{r.stderr}")
+    os.replace(tmp, lib)  # a library is there whole or not at all
     if verbose:
-        print(f"built {LIB}")
-    return LIB
+        print(f"built {lib}")
+    return lib
+
+
+def build(verbose: bool = True) -> str:
+    """Compiles every translation unit and links the shared library.  Always recompiles."""
+    return _build(LIB, SOURCES, verbose)
+
+
+def build_lm(verbose: bool = True) -> str:
+    """The part of the library that serves the token language models.  Always recompiles."""
+    return _build(LM_LIB, LM_SOURCES, verbose)
 
 
 if __name__ == "__main__":

@@ -112,3 +112,87 @@ def nano_config(preset: str = "A", max_secs: float = 240) -> Config:
     else:
         raise ValueError(f"unknown preset {preset!r}")
     return Config(model=m, data=DataConfig(max_secs=max_secs))
+
+
+# ---- token language models (vui_amd.lm): layers described one by one ----
+@dataclass
+class RotaryConfig:
+    """Rotation of the first `dims` entries of a vector, entry i paired with entry i + dims / 2, base^(-2 i / dims)."""
+
+    dims: int
+    base: float
+
+
+@dataclass
+class LatentAttentionConfig:
+    """Causal softmax attention over a cached latent per position.  Per head dim unrotated and rot_dim rotated query
+    and key dims and vdim value dims; kv_from names the layer whose latents are read instead of own ones."""
+
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+    rot: RotaryConfig
+    kv_from: int | None = None
+
+
+@dataclass
+class MinGRUConfig:
+    """Gated recurrence of `width` channels whose gate and candidate read the current token only."""
+
+    width: int
+
+
+@dataclass
+class GatedMLPConfig:
+    """Gated feed-forward with clamped branches."""
+
+    ff: int
+    limit: float
+
+
+@dataclass
+class LMLayerConfig:
+    mixer: "LatentAttentionConfig | MinGRUConfig"
+    mlp: GatedMLPConfig | None = None
+
+
+@dataclass
+class LMConfig:
+    """A decoder-only token model: config.json's `layers` (type, mixer, mlp), `norm.eps`, `vocab`, `width`."""
+
+    architecture: str
+    width: int
+    vocab: int
+    norm_eps: float
+    layers: "list[LMLayerConfig]"
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "LMConfig":
+        layers: "list[LMLayerConfig]" = []
+        for i, e in enumerate(d["layers"]):
+            mx = e["mixer"]
+            if e["type"] == "latent_attention":
+                mixer = LatentAttentionConfig(**{k: mx[k] for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "scale")},
+                                              rot=_from_dict(RotaryConfig, mx["rot"]), kv_from=mx.get("kv_from"))
+                if mixer.rot.dims > mixer.rot_dim or mixer.rot.dims % 2:
+                    raise ValueError(f"layer {i}: cannot rotate {mixer.rot.dims} of {mixer.rot_dim} dims")
+                if mixer.kv_from is not None:
+                    src = layers[mixer.kv_from].mixer if 0 <= mixer.kv_from < i else None
+                    if not isinstance(src, LatentAttentionConfig) or src.kv_from is not None:
+                        raise ValueError(f"layer {i}: kv_from={mixer.kv_from} names no earlier layer with latents of its own")
+                    if (src.kv_rank, src.rot_dim, src.rot) != (mixer.kv_rank, mixer.rot_dim, mixer.rot):
+                        raise ValueError(f"layer {i}: latents of layer {mixer.kv_from} have another shape or rotation")
+            elif e["type"] == "mingru":
+                mixer = MinGRUConfig(width=mx["width"])
+            else:
+                raise ValueError(f"layer {i}: unknown mixer {e['type']!r}")
+            mlp = None
+            if e.get("mlp") is not None:
+                if e["mlp"].get("kind", "dense") != "dense":
+                    raise ValueError(f"layer {i}: unknown feed-forward {e['mlp']['kind']!r}")
+                mlp = GatedMLPConfig(ff=e["mlp"]["ff"], limit=e["mlp"]["limit"])
+            layers.append(LMLayerConfig(mixer, mlp))
+        return cls(architecture=d["architecture"], width=d["width"], vocab=d["vocab"], norm_eps=d["norm"]["eps"], layers=layers)

@@ -9,15 +9,6 @@
 #include "internal.h"
 #include <hip/hip_ext.h>
 
-static thread_local char g_err[512] = "";
-
-void vui_set_error(const char* fmt, ...) {
-  va_list ap;
-  va_start(ap, fmt);
-  vsnprintf(g_err, sizeof(g_err), fmt, ap);
-  va_end(ap);
-}
-
 #define MAX_SPLITS 64
 
 // ---- scratch of the entry point that allocates nothing (vui_decode_attn_noalloc) ----
@@ -166,9 +157,6 @@ static size_t carve(const vui_config* c, int Bm, vui_ctx* x) {
 }
 
 extern "C" {
-
-const char* vui_last_error(void) { return g_err; }
-int vui_version(void) { return 1; }
 
 int64_t vui_workspace_bytes(const vui_config* cfg, int max_batch) {
   if (check_cfg(cfg, max_batch)) return VUI_EINVAL;
@@ -659,44 +647,6 @@ int vui_frame_step(vui_ctx* ctx, int64_t* codes_io, const int32_t* slot_idx, int
   return launch_frame_finish(codes_io, frames_out, B * c.n_quantizers, max_frames, frame_ctr, ctx->eos_prob,
                              eos_prob_out, B, stop ? stop->state : nullptr, stop ? stop->threshold : 0.f,
                              stop ? stop->min_frames : 0, st);
-}
-
-// ---- HIP graphs ----
-struct vui_graph {
-  hipGraph_t graph;
-  hipGraphExec_t exec;
-};
-
-int vui_graph_begin(vui_stream_t stream) {
-  HIP_TRY(hipStreamBeginCapture((hipStream_t)stream, hipStreamCaptureModeThreadLocal));
-  return VUI_OK;
-}
-
-int vui_graph_end(vui_stream_t stream, vui_graph** out) {
-  hipGraph_t g = nullptr;
-  HIP_TRY(hipStreamEndCapture((hipStream_t)stream, &g));
-  if (!out || !g) { if (g) (void)hipGraphDestroy(g); vui_set_error("capture produced no graph"); return VUI_EINVAL; }
-  hipGraphExec_t e = nullptr;
-  hipError_t err = hipGraphInstantiate(&e, g, nullptr, nullptr, 0);
-  if (err != hipSuccess) { (void)hipGraphDestroy(g); vui_set_error("hipGraphInstantiate failed: %s", hipGetErrorString(err)); return VUI_EHIP; }
-  vui_graph* vg = new (std::nothrow) vui_graph();
-  if (!vg) { (void)hipGraphExecDestroy(e); (void)hipGraphDestroy(g); vui_set_error("out of host memory"); return VUI_ENOMEM; }
-  vg->graph = g; vg->exec = e;
-  *out = vg;
-  return VUI_OK;
-}
-
-int vui_graph_launch(vui_graph* g, vui_stream_t stream) {
-  if (!g) { vui_set_error("NULL graph"); return VUI_EINVAL; }
-  HIP_TRY(hipGraphLaunch(g->exec, (hipStream_t)stream));
-  return VUI_OK;
-}
-
-void vui_graph_destroy(vui_graph* g) {
-  if (!g) return;
-  (void)hipGraphExecDestroy(g->exec);
-  (void)hipGraphDestroy(g->graph);
-  delete g;
 }
 
 // ---- single kernels ----

@@ -14,27 +14,18 @@
 // the norm, products of the rotation rounded before their sum, residual sums rounded).
 #include "common.h"
 #include "internal.h"
+#include "tile.h"
 #include <stdio.h>
 
-typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 pf_bf16x8;
-typedef __attribute__((__vector_size__(4 * sizeof(float)))) float pf_floatx4;
-union PfU128 { uint4 u; pf_bf16x8 v; };
-__device__ __forceinline__ pf_bf16x8 pf_frag(const uint4& x) { PfU128 t; t.u = x; return t.v; }
+typedef tl_bf16x8 pf_bf16x8;
+typedef tl_f32x4 pf_floatx4;
+__device__ __forceinline__ pf_bf16x8 pf_frag(const uint4& x) { return Tl<bf16_t>::frag(x); }
 
 enum { PF_BF16 = 0, PF_RESID = 1 };
 
-// Operand layout of the GEMMs ("tiled"): a matrix of R rows x K columns (K a multiple of 64, rows padded to 16) is
-// cut into blocks of 16 rows x 64 columns, block (r / 16, k / 64) at element offset ((r / 16) * (K / 64) + k / 64)
-// * 1024, and inside a block the 8-element piece p = (k % 16) / 8 of lane (r % 16) + 16 * ((k % 64) / 16) sits at
-// p * 512 + lane * 8.  A wave then fetches the operand fragment of a 16 x 64 block with two loads of 1 KiB
-// contiguous each (lane l: 16 bytes at 16 l), where the row-major form makes the 16 lanes of a quarter-wave read
-// 16 different lines - which the address unit serves at about a quarter of the rate (measured on this machine
-// from an L2-sized buffer: 9.6 TB/s over the chip for 16 rows x 64 bytes per instruction, 31 TB/s for 1 KiB
-// contiguous).  Weights are brought into this form once per context, activations are written in it by their
-// producers.
-__host__ __device__ __forceinline__ size_t pf_toff(int r, int k, int K) {
-  return ((size_t)(r >> 4) * (K >> 6) + (k >> 6)) * 1024 + (size_t)(((k & 15) >> 3) * 512 + (((k & 63) >> 4) * 16 + (r & 15)) * 8 + (k & 7));
-}
+// Both operands of the GEMMs are in the tiled layout of tile.h (blocks of 16 rows x 64 columns).  Weights are brought
+// into this form once per context, activations are written in it by their producers.
+__host__ __device__ __forceinline__ size_t pf_toff(int r, int k, int K) { return tl_off<bf16_t>(r, k, K); }
 
 struct PfGemm {
   const bf16_t* X;   // activations (M x K), tiled

@@ -1,0 +1,62 @@
+// Gated recurrence S_t = a_t S_(t-1) + b_t over the positions of one sequence, channel by channel, fp32 throughout;
+// output S_t * gate_t in the tiled operand layout.  (a, b) pairs come from the projection's epilogue.
+//
+// The positions are cut into chunks of 32: one launch folds every chunk to its (product of a, end value from zero),
+// the second starts each chunk from the fold of the chunks before it.  The incoming state is copied next to the folds
+// first, because the last chunk's workgroup overwrites it while others still start from it.
+#include "common.h"
+#include "lm.h"
+#include "tile.h"
+
+__global__ __launch_bounds__(256) void scan_fold_kernel(const ScanArgs p, int nchunks) {
+  const int ch = blockIdx.x * 256 + threadIdx.x, c = blockIdx.y;
+  if (ch >= p.W) return;
+  if (c == nchunks) {  // the state the sequence starts from
+    p.agg[(size_t)nchunks * p.ld + ch] = make_float2(0.f, p.from_zero ? 0.f : p.state[ch]);
+    return;
+  }
+  const int t1 = min((c + 1) * LM_SCAN_CHUNK, p.T);
+  float a = 1.f, b = 0.f;
+#pragma unroll 8
+  for (int t = c * LM_SCAN_CHUNK; t < t1; ++t) {
+    const float2 u = p.upd[(size_t)t * p.ld + ch];
+    b = fmaf(u.x, b, u.y);
+    a *= u.x;
+  }
+  p.agg[(size_t)c * p.ld + ch] = make_float2(a, b);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void scan_apply_kernel(const ScanArgs p, int nchunks) {
+  const int ch = blockIdx.x * 256 + threadIdx.x, c = blockIdx.y;
+  if (ch >= p.W) return;
+  float s;
+  if (nchunks == 1) {
+    s = p.from_zero ? 0.f : p.state[ch];
+  } else {
+    s = p.agg[(size_t)nchunks * p.ld + ch].y;
+    for (int k = 0; k < c; ++k) {
+      const float2 g = p.agg[(size_t)k * p.ld + ch];
+      s = fmaf(g.x, s, g.y);
+    }
+  }
+  const int t1 = min((c + 1) * LM_SCAN_CHUNK, p.T);
+#pragma unroll 8
+  for (int t = c * LM_SCAN_CHUNK; t < t1; ++t) {
+    const float2 u = p.upd[(size_t)t * p.ld + ch];
+    s = fmaf(u.x, s, u.y);
+    El<T>::st((T*)p.act + tl_off<T>(t, ch, p.out_k), s * El<T>::ld((const T*)p.gate + (size_t)t * p.ld + ch));
+  }
+  if (c == nchunks - 1) p.state[ch] = s;
+}
+
+int launch_gated_scan(const ScanArgs& a, hipStream_t st) {
+  if (a.T < 1 || a.W < 1 || a.ld < a.W) { vui_set_error("gated scan: bad shape T=%d W=%d", a.T, a.W); return VUI_EINVAL; }
+  const int nchunks = (a.T + LM_SCAN_CHUNK - 1) / LM_SCAN_CHUNK;
+  const int gx = (a.W + 255) / 256;
+  if (nchunks > 1) hipLaunchKernelGGL(scan_fold_kernel, dim3(gx, nchunks + 1), dim3(256), 0, st, a, nchunks);
+  if (a.dtype == VUI_DTYPE_F32) hipLaunchKernelGGL(scan_apply_kernel<float>, dim3(gx, nchunks), dim3(256), 0, st, a, nchunks);
+  else hipLaunchKernelGGL(scan_apply_kernel<bf16_t>, dim3(gx, nchunks), dim3(256), 0, st, a, nchunks);
+  HIP_TRY(hipGetLastError());
+  return VUI_OK;
+}

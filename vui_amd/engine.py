@@ -16,7 +16,8 @@ import torch
 from torch import Tensor
 
 from . import _lib
-from .model import MAX_BATCH, Graph, SampleDev, Vui, make_sample_params
+from .model import MAX_BATCH, Graph, SampleDev, Vui, make_sample_params  # noqa: F401
+from .slots import SlotEngine, _get_bucket, _make_buckets  # noqa: F401
 
 FRAME_RATE = 12.5  # codec frames per second (src/vui/qwen_codec.py:27-30)
 DEFAULT_WPS = 3.0  # words per second when the prompt gives none (src/vui/engine.py:41)
@@ -102,24 +103,6 @@ class _ActiveSlot:
     max_turn_frames: int = 0
     seq_offset: int = 0
     last_codes: Tensor | None = None
-
-
-def _make_buckets(max_bs: int) -> list[int]:
-    """src/vui/engine.py:134-142."""
-    buckets, b = [], 1
-    while b < max_bs:
-        buckets.append(b)
-        b *= 2
-    if not buckets or buckets[-1] != max_bs:
-        buckets.append(max_bs)
-    return buckets
-
-
-def _get_bucket(batch_size: int, buckets: list[int]) -> int:
-    for b in buckets:
-        if batch_size <= b:
-            return b
-    return buckets[-1]
 
 
 class Row:
@@ -269,7 +252,7 @@ class Row:
 _CU_STREAMS: dict = {}  # (device, first compute unit, count) -> stream bound to that range (never destroyed)
 
 
-class Engine:
+class Engine(SlotEngine):
     """Streaming (B=1) and batched (B=N) decode over one flash-style KV cache."""
 
     def __init__(self, name: str | None = None, *, model: Vui | None = None, codec=None, max_rows: int = 1,
@@ -278,8 +261,7 @@ class Engine:
             if name is None:
                 raise ValueError("pass model= or a local checkpoint path")
             model = Vui.from_pretrained_inf(name)
-        if max_rows < 1 or max_rows > MAX_BATCH:
-            raise ValueError(f"max_rows must be in [1, {MAX_BATCH}]")
+        self._check_rows(max_rows)
         self.model = model
         self.codec = codec
         self.max_rows = max_rows
@@ -297,10 +279,8 @@ class Engine:
         self._sc_emb = None
         if sc_token_id is not None:
             self._sc_emb = model.token_emb(torch.tensor([[sc_token_id]], device=self.device)).to(self.dtype)
+        self._setup_slots(self.CS)
         self._setup_graphs()
-        self._setup_rep_state()
-        self._free: set[int] = set(range(max_rows))
-        self._rows: dict[int, Row] = {}
         self._frame_graphs: dict = {}
         self._lane_streams: list = []
         self._split = None
@@ -349,8 +329,6 @@ class Engine:
         model, dev, dt = self.model, self.device, self.dtype
         model.decoder.allocate_flash_kv_cache(self.max_rows + 1, dev, dt, max_seqlen=self.max_seq)
         self.seq_lens = model.decoder.flash_kv_caches[0].seq_lens
-        self._pad_slot = self.max_rows
-        self._buckets = _make_buckets(self.max_rows)
         rq_batch_sizes = tuple(sorted(set(self._buckets) | {1, self.max_rows}))
         model.rq_transformer.setup_cuda_graph_kv(dev, dt, top_k=100, batch_sizes=rq_batch_sizes)
         self._zero_rq_bias = torch.zeros(self.Q - 1, self.CS, device=dev, dtype=torch.float32)
@@ -365,9 +343,6 @@ class Engine:
         self._gc_hidden_out = torch.zeros(B_max, self.D, device=dev, dtype=dt)
         self._gc_cb0_out = torch.zeros(B_max, self.CS, device=dev, dtype=dt)
         self._gc_eos_out = torch.zeros(B_max, 1, device=dev, dtype=dt)
-        self._g_slot_idx = torch.full((B_max,), self._pad_slot, device=dev, dtype=torch.int32)
-        self._g_seq_inc = torch.zeros(self.max_rows + 1, device=dev, dtype=torch.int32)
-        self._bucketed_graphs: dict[int, Graph] = {}
         # fused frame state
         self._frame_ctr = torch.zeros(1, dtype=torch.int32, device=dev)
         self._code0 = torch.zeros(N, dtype=torch.long, device=dev)
@@ -387,15 +362,6 @@ class Engine:
         self.model.decoder._step(codes=self._g_codes_in, emb=None, slot_idx=None, seq_inc=None, B=B,
                                  hidden_out=self._g_hidden_out, cb0_out=self._g_cb0_out, eos_out=self._g_eos_out,
                                  n_splits=self._splits(B), stream=stream)
-
-    def _capture(self, body) -> Graph:
-        """Warm once and capture; warm-up and capture advance seq_lens, so it is restored
-        (src/vui/engine.py:451-471)."""
-        saved = self.seq_lens.clone()
-        g = Graph(self.model, body, warmup=1)
-        torch.cuda.current_stream().synchronize()
-        self.seq_lens.copy_(saved)
-        return g
 
     def _decode_step(self) -> tuple[Tensor, Tensor, Tensor]:
         """Replay the batched backbone graph; returns views of the static (hidden, cb0, eos)
@@ -422,44 +388,13 @@ class Engine:
                                  stream=stream)
 
     def _bucketed_decode_step(self, B_active: int) -> tuple[Tensor, Tensor, Tensor]:
-        """src/vui/engine.py:525-534: pad the active rows up to the bucket with rows that write to the
-        padding slot, replay that bucket's graph."""
-        B_bucket = _get_bucket(B_active, self._buckets)
-        self._g_slot_idx[B_active:B_bucket].fill_(self._pad_slot)
-        g = self._bucketed_graphs.get(B_bucket)
-        if g is None:
-            saved_idx, saved_inc = self._g_slot_idx.clone(), self._g_seq_inc.clone()
-            self._g_slot_idx[:B_bucket].fill_(self._pad_slot)
-            self._g_seq_inc.zero_()
-            g = self._capture(lambda st: self._backbone_decode_body_b(B_bucket, st))
-            self._g_slot_idx.copy_(saved_idx)
-            self._g_seq_inc.copy_(saved_inc)
-            self._bucketed_graphs[B_bucket] = g
-        g.replay()
+        """src/vui/engine.py:525-534: see SlotEngine._replay_bucket."""
+        self._replay_bucket(B_active, self._backbone_decode_body_b)
         return self._gc_hidden_out[:B_active], self._gc_cb0_out[:B_active], self._gc_eos_out[:B_active]
 
     # ------------------------------------------------------------------ repetition penalty
-    def _setup_rep_state(self) -> None:
-        """Device-resident rolling counts (src/vui/engine.py:540-553); the ring position lives on the
-        device too so that the sampler can run inside a captured graph."""
-        N = self.max_rows
-        self._rep_counts = torch.zeros(N, self.CS, device=self.device, dtype=torch.float32)
-        self._rep_history: Tensor | None = None
-        self._rep_pos = torch.zeros(N, 2, device=self.device, dtype=torch.int32)
-        self._rep_window_cur = 0
-
-    def _rep_reset(self, penalty: float, window: int) -> None:
-        """src/vui/engine.py:555-569."""
-        self._rep_counts.zero_()
-        self._rep_pos.zero_()
-        if penalty <= 1.0:
-            return
-        if window > 0 and (self._rep_history is None or self._rep_window_cur != window):
-            self._rep_history = torch.zeros(self.max_rows, window, device=self.device, dtype=torch.int32)
-            self._rep_window_cur = window
-            self._frame_graphs = {}
-        elif window > 0:
-            self._rep_history.zero_()
+    def _rep_window_changed(self) -> None:
+        self._frame_graphs = {}
 
     def _sample_cb0(self, logits: Tensor, cfg: GenConfig, *, top_k: int | None = -1, frame_ctr: Tensor | None = None,
                     out: Tensor | None = None) -> Tensor:
@@ -480,19 +415,11 @@ class Engine:
         return out
 
     # ------------------------------------------------------------------ rows
-    def new_row(self) -> Row:
-        if not self._free:
-            raise RuntimeError(f"No free rows (max_rows={self.max_rows} all in use)")
-        idx = min(self._free)
-        self._free.remove(idx)
-        row = Row(self, idx)
-        self._rows[idx] = row
-        self.seq_lens[idx] = 0
-        return row
+    def _make_row(self, idx: int) -> Row:
+        return Row(self, idx)
 
     def _release_row(self, row: Row) -> None:
-        self._rows.pop(row.idx, None)
-        self._free.add(row.idx)
+        super()._release_row(row)
         if row._codec_ctx is not None:
             row._codec_ctx.reset()
 
@@ -506,11 +433,6 @@ class Engine:
         codes_t = frame_codes.unsqueeze(0).unsqueeze(-1)
         decode_codes = codes_t[:, :n_codebooks] if n_codebooks > 0 else codes_t
         return row._codec_ctx.decode_frame(decode_codes, store_codes=codes_t)
-
-    def reset(self) -> None:
-        for row in list(self._rows.values()):
-            row.close()
-        self.seq_lens.zero_()
 
     def _rewind_row(self, row: Row, offset: int) -> int:
         """KV rewind = overwrite one int32; K/V beyond it are never cleared (engine.py:651-654)."""
@@ -1026,11 +948,8 @@ class Engine:
             B_active = len(slot_list)
             B_bucket = _get_bucket(B_active, self._buckets)
             if slot_list != prev_slots:  # membership changes only when a request ends or starts
-                slots_t = torch.tensor(slot_list, dtype=torch.int32, device=self.device)
+                slots_t = self._set_active_slots(slot_list)
                 slots_l = slots_t.long()
-                self._g_slot_idx[:B_active] = slots_t
-                self._g_seq_inc.zero_()
-                self._g_seq_inc[slots_l] = 1
                 prev_slots = slot_list
             torch.index_select(last, 0, slots_l, out=self._gc_codes_in[:B_active])
             hidden_all, cb0_all, eos_all = self._bucketed_decode_step(B_active)

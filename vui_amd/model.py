@@ -18,6 +18,7 @@ from torch import Tensor
 
 from . import _lib
 from .config import Config, VuiConfig
+from .registry import register_model
 
 MAX_BATCH = _lib.VUI_MAX_BATCH
 
@@ -209,7 +210,7 @@ class Graph:
     """A captured HIP graph of native calls (stands for torch.cuda.CUDAGraph in the reference)."""
 
     def __init__(self, model: "Vui", fn, warmup: int = 1):
-        lib = _lib.load()
+        lib = _lib.load(lm_only=True)
         s = model._cap_stream
         s.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(s):
@@ -525,6 +526,7 @@ class RQTransformer:
         return self._gkv_codes_out[:B, :Q]
 
 
+@register_model("Vui")
 class Vui:
     """Model shell.  Mirrors Vui in src/vui/model.py:1054-1311 for inference."""
 
