@@ -51,7 +51,7 @@ typedef struct vui_lm_layer {
   const void* w_in;       /* (in_rows, w64) tiled: everything that reads h; row order in vui_amd/lm_layout.py */
   const void* w_out;      /* (out_rows, out_k) tiled: mixer and feed-forward output side by side along k */
   const void* w_uk_t;     /* (heads, rank16, dim64) tiled: per head, latent <- unrotated query */
-  const void* w_uk;       /* (heads, dim16, rank64) tiled: per head, key <- latent (bf16 contexts) */
+  const void* w_uk;       /* (heads, dim64, rank64) tiled: per head, key <- latent (bf16 contexts) */
   const void* w_uv;       /* (heads, vdim16, rank64) tiled: per head, value <- latent */
   const float* latent_norm; /* (rank16) */
   const float* rope;      /* (max_seqlen, rot_pairs, 2) cos/sin */

@@ -235,7 +235,7 @@ static int lm_attention(vui_lm_ctx* x, int l, int M, const LmRows& rows, LmGemm&
     memset(&k, 0, sizeof(k));
     k.X = (const char*)L.c_cache + (size_t)rows.slot * d.s64 * d.rank64 * e;
     k.M = rows.pos0 + M; k.K = d.rank64; k.d = d; k.rows = rows;
-    k.W = L.w_uk; k.N = d.dim16; k.wz = (size_t)d.dim16 * d.rank64; k.kv_out = x->kx; k.kv_z = (size_t)d.s64 * d.dim64;
+    k.W = L.w_uk; k.N = d.dim64; k.wz = (size_t)d.dim64 * d.rank64; k.kv_out = x->kx; k.kv_z = (size_t)d.s64 * d.dim64;
     if ((rc = launch_lm_gemm(c.dtype, LM_EXPAND_K, k, L.heads, st))) return rc;
     k.W = L.w_uv; k.N = d.vdim16; k.wz = (size_t)d.vdim16 * d.rank64; k.kv_out = x->vx; k.kv_z = (size_t)d.s64 * d.vdim16;
     if ((rc = launch_lm_gemm(c.dtype, LM_EXPAND_V, k, L.heads, st))) return rc;

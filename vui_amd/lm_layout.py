@@ -72,10 +72,11 @@ def latent_attention_weights(w: dict, p: str, mx, d) -> dict:
     o = w[m + "o"].reshape(-1, H, mx.vdim)
     o_pad = torch.zeros(o.shape[0], H, d.vdim16, dtype=o.dtype, device=o.device)
     o_pad[:, :, :mx.vdim] = o
+    # expanded keys get all dim64 columns: the pad columns of the query operand hold whatever another layer left there
     out = {
         "mix": torch.cat(parts), "out": o_pad.reshape(o.shape[0], H * d.vdim16),
         "w_uk_t": torch.cat([tile(pad_to(uk[h].T, d.rank16, d.dim64)) for h in range(H)]),
-        "w_uk": torch.cat([tile(pad_to(uk[h], d.dim16, d.rank64)) for h in range(H)]),
+        "w_uk": torch.cat([tile(pad_to(uk[h], d.dim64, d.rank64)) for h in range(H)]),
         "w_uv": torch.cat([tile(pad_to(uv[h], d.vdim16, d.rank64)) for h in range(H)]),
     }
     if mx.kv_from is None:
