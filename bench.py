@@ -514,6 +514,116 @@ def serve_line(sd, preset="A", n_requests=32, max_rows=16, int8=False):
             "wall_s": round(dt, 3), "aggregate_frames_per_s": round(n_frames / dt, 1), "rtf_aggregate": round(n_frames / dt / 12.5, 1)}
 
 
+# Sizes of the token-model lines: (name, width, heads, ff, dim, rot_dim, vdim, kv_rank, layers).  The Vui backbone
+# beside each has the same width, heads, feed-forward and layer count (full attention over heads x width / heads).
+LM_SIZES = [("w768", 768, 8, 2048, 64, 32, 96, 256, 8), ("w1024", 1024, 8, 2816, 128, 64, 128, 512, 8),
+            ("w2048", 2048, 16, 4096, 128, 64, 128, 512, 8)]
+
+
+def lm_work(cfg, L: float, B: int):
+    """(bytes of one decode step of B rows at cache length L, flops of its weights per token, flops of attention per
+    token and visible key in the expanded form).  Every weight, latent, key part and state once, bf16."""
+    W = cfg["width"]
+    wb = W * cfg["vocab"]
+    cache = state = attn = 0
+    for layer in cfg["layers"]:
+        mx = layer["mixer"]
+        if layer["type"] == "latent_attention":
+            H, r = mx["heads"], mx["kv_rank"]
+            wb += W * (H * (mx["dim"] + mx["rot_dim"]) + (0 if "kv_from" in mx else r + mx["rot_dim"]) + H + H * mx["vdim"]) + H * r * (mx["dim"] + mx["vdim"])
+            cache += (r + mx["rot_dim"]) * 2
+            attn += 2 * H * (mx["dim"] + mx["rot_dim"] + mx["vdim"])
+        else:
+            wb += 4 * W * mx["width"]
+            state += 8 * mx["width"]
+        wb += 3 * W * layer["mlp"]["ff"]
+    return wb * 2 + B * (cache * L + state), 2 * (wb - W * cfg["vocab"]), attn
+
+
+def lm_lines(sizes=None, batches=(1, 4, 16), prompts=(512, 2048), L=1024, which="both"):
+    """Token models with random weights at sizes that resemble a real model's layers: prefill of one prompt and the
+    decode step of B rows at cache length L from its captured graph, beside the Vui backbone of equal size (prompt pass
+    and backbone step)."""
+    import torch
+
+    from vui_amd.config import Config, DataConfig, VuiConfig
+    from vui_amd.engine import Engine
+    from vui_amd.lm import TokenLM
+    from vui_amd.lm_engine import TokenEngine
+    from vui_amd.model import Vui
+    from vui_amd.synthetic import synthetic_state_dict, token_lm_config, token_lm_state_dict
+
+    def timed(fn, n):
+        fn()
+        torch.cuda.synchronize()
+        e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+        e0.record()
+        for _ in range(n):
+            fn()
+        e1.record()
+        torch.cuda.synchronize()
+        return e0.elapsed_time(e1) * 1e3 / n
+
+    S = 2304
+    for name, W, H, F, dim, rot, vdim, rank, nl in LM_SIZES:
+        if sizes and name not in sizes:
+            continue
+        out = {"config": f"token_lm_{name}", "dtype": "bf16", "data": "synthetic", "layers": nl, "width": W, "heads": H, "ff": F, "kv_rank": rank}
+        if which in ("both", "lm"):
+            cfg = token_lm_config(W, H, F, dim, rot, vdim, rank, nl, vocab=2048)
+            eng = TokenEngine(model=TokenLM.from_config(cfg, token_lm_state_dict(cfg, 0, "cuda"), max_seqlen=S), max_rows=16)
+            m = eng.model
+            for t in m.cache.c.values():
+                t.normal_()
+            for t in m.cache.kr.values():
+                t.normal_()
+            toks = torch.randint(0, cfg["vocab"], (S,), device="cuda")
+            for T in prompts:
+                us = timed(lambda: m.prefill(toks[:T], 0, 0, [T - 1]), 5)
+                _, fl, at = lm_work(cfg, 0, 1)
+                fl = fl * T + at * T * (T + 1) / 2
+                out[f"prefill_{T}"] = {"ms": round(us / 1e3, 3), "tokens_per_s": round(T * 1e6 / us), "TFLOPs": round(fl / us / 1e6, 1), "mfma_frac": round(fl / us / 1e6 / 2500, 4)}
+            for B in batches:
+                eng._set_active_slots(list(range(B)))
+                eng.seq_lens.fill_(L - 26)
+                eng._g_tokens[:B] = toks[:B]
+                us = timed(lambda: eng._replay_bucket(B, eng._decode_body), 50)
+                by, _, _ = lm_work(cfg, L, B)
+                out[f"decode_b{B}"] = {"us": round(us, 1), "tokens_per_s": round(B * 1e6 / us), "GBs": round(by / us / 1e3, 1), "hbm_frac": round(by / us / 1e3 / HBM_PEAK_GBS, 4)}
+            del eng, m
+        if which in ("both", "vui"):
+            c = VuiConfig(d_model=W, n_layers=nl, n_heads=H, intermediate_size=F, n_quantizers=16, codebook_size=2048, use_rq_transformer=True,
+                          rq_d_model=512, rq_n_layers=4, rq_n_heads=8, vocab_size=512, max_text_tokens=S - 16, max_audio_tokens=0)
+            vm = Vui(Config(model=c, data=DataConfig(max_secs=0)), synthetic_state_dict(c, 0), dtype=torch.bfloat16)
+            vui = {"forms": {}}
+            wl = nl * (4 * W * W + 3 * W * F)
+            for B in batches:
+                ve = Engine(model=vm, max_rows=B, max_seq=S)
+                vm.decoder._k.normal_()
+                vm.decoder._v.normal_()
+                ve._decode_step()
+                ve.seq_lens.fill_(L - 26)
+                us = timed(ve._decode_graph.replay, 50)
+                vm._native.status()
+                by = (wl + W * 2048) * 2 + B * L * nl * 4 * W
+                vui[f"decode_b{B}"] = {"us": round(us, 1), "tokens_per_s": round(B * 1e6 / us), "GBs": round(by / us / 1e3, 1), "hbm_frac": round(by / us / 1e3 / HBM_PEAK_GBS, 4)}
+                vui["forms"][f"b{B}"] = "one launch" if (vm._native.fused(-1) if B == 1 else vm._native.bb_batch()) else "kernel sequence"
+                if B == batches[0]:
+                    emb = (torch.randn(1, max(prompts), W, device="cuda") * 0.1).to(torch.bfloat16)
+                    for T in prompts:
+                        def pre():
+                            ve.seq_lens[0] = 0
+                            vm.decoder.forward_flash(emb[:, :T], None, slot_idx=None, known=(0, 0))
+                        us = timed(pre, 5)
+                        fl = 2 * wl * T + nl * 4 * W * T * (T + 1) / 2
+                        vui[f"prefill_{T}"] = {"ms": round(us / 1e3, 3), "tokens_per_s": round(T * 1e6 / us), "TFLOPs": round(fl / us / 1e6, 1), "mfma_frac": round(fl / us / 1e6 / 2500, 4)}
+                del ve
+            out["vui_backbone"] = vui
+            del vm
+        torch.cuda.empty_cache()
+        yield out
+
+
 def copy_line():
     """The practical bandwidth ceiling of the box: a plain 1 GiB device-to-device copy (reads + writes)."""
     import torch
@@ -748,6 +858,11 @@ def main():
                     help="print only the vocoder line (the run rocprofv3 summaries of the vocoder kernels come from)")
     ap.add_argument("--split-audio-only", action="store_true",
                     help="print only the streamed turn with audio on a divided GPU (the run its rocprofv3 summary comes from)")
+    ap.add_argument("--lm", nargs="*", metavar="SIZE", default=None,
+                    help="print only the token-model lines (sizes: w768 w1024 w2048; none named: all), each beside the Vui backbone of equal size")
+    ap.add_argument("--lm-which", default="both", choices=["both", "lm", "vui"], help="one side of the --lm lines (for profiles)")
+    ap.add_argument("--lm-batch", type=int, nargs="*", default=[1, 4, 16], help="rows of the --lm decode steps")
+    ap.add_argument("--lm-prompt", type=int, nargs="*", default=[512, 2048], help="prompt lengths of the --lm lines")
     ap.add_argument("--phase-clock", action="store_true",
                     help="print the phase stamps of one workgroup of the batch-1 frame kernel (with --int8: int8 weights)")
     ap.add_argument("--bb-phase-clock", type=int, default=0, metavar="ROWS",
@@ -760,6 +875,10 @@ def main():
         print("bench.py measures one GPU: this path has no multi-GPU part (streams are independent); "
               "run with --gpus 1", file=sys.stderr)
         sys.exit(2)
+    if args.lm is not None:
+        for ln in lm_lines(args.lm, args.lm_batch, args.lm_prompt, which=args.lm_which):
+            print(json.dumps(ln), flush=True)
+        return
     if args.phase_clock:
         return phase_clock(args)
     if args.bb_phase_clock:

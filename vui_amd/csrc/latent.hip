@@ -146,11 +146,131 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs p) {
     }
     __syncthreads();
   }
-  float* out = p.part + (((size_t)m * p.heads + h) * p.n_splits + sp) * (R + 2);
-  if (tid == 0) { out[0] = M; out[1] = L; }
+  const size_t piece = ((size_t)m * p.heads + h) * p.n_splits + sp;
+  if (tid == 0) *reinterpret_cast<float2*>(p.part_ml + 2 * piece) = make_float2(M, L);
 #pragma unroll
   for (int i = 0; i < LAT_ACC; ++i)
-    if (tid + 256 * i < R) out[2 + tid + 256 * i] = acc[i];
+    if (tid + 256 * i < R) p.part[piece * R + tid + 256 * i] = acc[i];
+}
+
+// ---- attention in the latent space on the matrix cores (bf16): one workgroup per (row, 16 heads, split) ----
+// All heads read the same latents, so 32 keys are staged in LDS once and serve 16 heads.  Scores^T (keys x heads) =
+// [c | k_rot] [q_lat | q_rot]^T, the four waves dealing key tile and half of the columns between them; every wave then
+// has all scores of its lane's head and averages a quarter of the latent columns: out^T (columns x heads) = C^T p^T,
+// the weights as a bf16 pair (value and remainder).  The transposed operand is gathered from LDS element by element.
+// RK = rank64 / 64, RB = rot32 / 32.
+template <int RK, int RB>
+__global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const LatentArgs p) {
+  constexpr int NC = 2 * RK + RB;         // 32-column chunks of a key row
+  constexpr int NQ = (NC + 1) / 2;        // chunks per wave
+  constexpr int CT = RK * 2048, RT = RB * 1024;  // elements of the staged tiles (32 keys)
+  extern __shared__ __align__(16) bf16_t tile[];  // 2 x (CT + RT)
+  __shared__ __align__(16) float sco[4][64 * 4];
+  const int m = blockIdx.x, sp = blockIdx.z, tid = threadIdx.x;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, l16 = lane & 15, kg = lane >> 4;
+  const int t = wave & 1, half = wave >> 1;
+  const int head = blockIdx.y * 16 + l16, hq = min(head, p.heads - 1);
+  const int slot = lm_slot(p.rows, m);
+  const int len = min(max(lm_pos(p.rows, m, slot) + 1, 1), p.rows.S);
+  int lo, hi;
+  latent_range(len, p.n_splits, sp, lo, hi);
+  const uint4* cc = reinterpret_cast<const uint4*>((const bf16_t*)p.c_cache + (size_t)slot * p.d.s64 * (RK * 64));
+  const uint4* kc = reinterpret_cast<const uint4*>((const bf16_t*)p.kr_cache + (size_t)slot * p.d.s64 * (RB * 32));
+  // 32 keys are one contiguous run of either cache
+  uint4 rc[RK], rr = make_uint4(0, 0, 0, 0);
+  auto fetch = [&](int j0) {
+#pragma unroll
+    for (int i = 0; i < RK; ++i) rc[i] = cc[(size_t)(j0 >> 5) * (CT / 8) + tid + 256 * i];
+    rr = kc[(size_t)(j0 >> 5) * (RT / 8) + min(tid, RT / 8 - 1)];
+  };
+  auto stage = [&](bf16_t* dst) {
+    uint4* d = reinterpret_cast<uint4*>(dst);
+#pragma unroll
+    for (int i = 0; i < RK; ++i) d[tid + 256 * i] = rc[i];
+    if (tid < RT / 8) d[CT / 8 + tid] = rr;
+  };
+  if (lo < hi) fetch(lo);
+  uint4 qf[NQ];
+#pragma unroll
+  for (int i = 0; i < NQ; ++i) {
+    const int c = min(2 * i + half, NC - 1);
+    const bf16_t* src = c < 2 * RK
+        ? (const bf16_t*)p.qlat + hq * p.qlat_z + ((size_t)(m >> 4) * RK + (c >> 1)) * 1024 + (c & 1) * 512 + ((m & 15) + 16 * kg) * 8
+        : (const bf16_t*)p.qr + hq * p.qr_z + ((size_t)(m >> 4) * RB + (c - 2 * RK)) * 512 + ((m & 15) + 16 * kg) * 8;
+    qf[i] = *reinterpret_cast<const uint4*>(src);
+  }
+  tl_f32x4 acc[RK];
+#pragma unroll
+  for (int i = 0; i < RK; ++i) acc[i] = tl_f32x4{0.f, 0.f, 0.f, 0.f};
+  float m_run = -INFINITY, l_run = 0.f;
+  if (lo < hi) stage(tile);
+  __syncthreads();
+  int buf = 0;
+  for (int j0 = lo; j0 < hi; j0 += 32) {
+    const bf16_t* cur = tile + buf * (CT + RT);
+    const bool more = j0 + 32 < hi;
+    if (more) fetch(j0 + 32);
+    tl_f32x4 s = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < NQ; ++i) {
+      const int c = 2 * i + half;
+      if (c < NC) {  // uniform over the wave
+        const bf16_t* a = c < 2 * RK ? cur + (t * RK + (c >> 1)) * 1024 + (c & 1) * 512 : cur + CT + (t * RB + (c - 2 * RK)) * 512;
+        s = Tl<bf16_t>::mma(*reinterpret_cast<const uint4*>(a + lane * 8), qf[i], s);
+      }
+    }
+    *reinterpret_cast<tl_f32x4*>(&sco[half * 2 + t][lane * 4]) = s;
+    __syncthreads();
+    // keys j0 + 16 u + 4 kg + r of this lane's head
+    float sv[8], mx = -INFINITY;
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const tl_f32x4 a = *reinterpret_cast<const tl_f32x4*>(&sco[u][lane * 4]) + *reinterpret_cast<const tl_f32x4*>(&sco[2 + u][lane * 4]);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float v = j0 + 16 * u + 4 * kg + r < hi ? a[r] * p.scale : -INFINITY;
+        sv[4 * u + r] = v;
+        mx = fmaxf(mx, v);
+      }
+    }
+    mx = rows_max(mx);
+    const float m_new = fmaxf(m_run, mx);  // finite: key j0 is in range
+    const float alpha = expf(m_run - m_new);
+    float pv[8], ps = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) { pv[e] = expf(sv[e] - m_new); ps += pv[e]; }
+    l_run = l_run * alpha + ps;
+    m_run = m_new;
+    uint4 hi4, lo4;
+    hi4.x = f2bf2(pv[0], pv[1]); hi4.y = f2bf2(pv[2], pv[3]); hi4.z = f2bf2(pv[4], pv[5]); hi4.w = f2bf2(pv[6], pv[7]);
+    lo4.x = f2bf2(pv[0] - bf_lo(hi4.x), pv[1] - bf_hi(hi4.x)); lo4.y = f2bf2(pv[2] - bf_lo(hi4.y), pv[3] - bf_hi(hi4.y));
+    lo4.z = f2bf2(pv[4] - bf_lo(hi4.z), pv[5] - bf_hi(hi4.z)); lo4.w = f2bf2(pv[6] - bf_lo(hi4.w), pv[7] - bf_hi(hi4.w));
+#pragma unroll
+    for (int i = 0; i < RK; ++i) {
+      // 16 columns of block i, column group `wave`: column l16, the lane's eight keys
+      const bf16_t* q = cur + i * 1024 + (l16 >> 3) * 512 + (4 * kg + 16 * wave) * 8 + (l16 & 7);
+      uint4 v;
+      v.x = (uint32_t)q[0] | ((uint32_t)q[8] << 16);
+      v.y = (uint32_t)q[16] | ((uint32_t)q[24] << 16);
+      const bf16_t* q1 = q + RK * 1024;
+      v.z = (uint32_t)q1[0] | ((uint32_t)q1[8] << 16);
+      v.w = (uint32_t)q1[16] | ((uint32_t)q1[24] << 16);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) acc[i][r] *= alpha;
+      acc[i] = Tl<bf16_t>::mma(v, hi4, acc[i]);
+      acc[i] = Tl<bf16_t>::mma(v, lo4, acc[i]);
+    }
+    if (more) stage(tile + (buf ^ 1) * (CT + RT));
+    __syncthreads();
+    buf ^= 1;
+  }
+  l_run = rows_sum(l_run);
+  if (head >= p.heads) return;
+  const size_t piece = ((size_t)m * p.heads + head) * p.n_splits + sp;
+  if (wave == 0 && kg == 0) *reinterpret_cast<float2*>(p.part_ml + 2 * piece) = make_float2(m_run, l_run);
+#pragma unroll
+  for (int i = 0; i < RK; ++i)
+    *reinterpret_cast<tl_f32x4*>(p.part + piece * (RK * 64) + i * 64 + wave * 16 + 4 * kg) = acc[i];
 }
 
 // ---- merge of the pieces, value expansion through W_uv[h], head gate: 16 rows x up to 64 value dims of one head ----
@@ -161,19 +281,33 @@ __global__ __launch_bounds__(256) void latent_value_kernel(const LatentArgs p) {
   constexpr int EP = Tl<T>::EP, P = 16 / EP;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int h = blockIdx.x, mt = blockIdx.z, R = p.d.rank64, ns = p.n_splits;
-  for (int r = wave; r < 16; r += 4) {
-    const int m = mt * 16 + r;
-    const float* pc = p.part + ((size_t)min(m, p.M - 1) * p.heads + h) * ns * (R + 2);
-    const float ms = lane < ns ? pc[(size_t)lane * (R + 2)] : -INFINITY;
-    const float ls = lane < ns ? pc[(size_t)lane * (R + 2) + 1] : 0.f;
+  const int nrow = min(16, p.M - mt * 16), ncol = (R + 255) / 256;
+  for (int it = wave; it < nrow * ncol; it += 4) {  // a wave merges 256 columns of a row
+    const int r = it / ncol, k = (it - r * ncol) * 256 + 4 * lane;
+    const size_t piece = ((size_t)(mt * 16 + r) * p.heads + h) * ns;
+    const float2 ml = *reinterpret_cast<const float2*>(p.part_ml + 2 * (piece + min(lane, ns - 1)));
+    const float* pc = p.part + piece * R + min(k, R - 4);
+    const float ms = lane < ns ? ml.x : -INFINITY;
     const float M = wave_max(ms);
     float w = ms == -INFINITY ? 0.f : expf(ms - M);
-    const float L = wave_sum(w * ls);
-    w /= L;
-    for (int k = lane; k < R; k += 64) {
-      float a = 0.f;
-      for (int s = 0; s < ns; ++s) a = fmaf(__shfl(w, s), pc[(size_t)s * (R + 2) + 2 + k], a);
-      El<T>::st(xs + tl_off<T>(r, k, R), m < p.M ? a : 0.f);
+    w /= wave_sum(lane < ns ? w * ml.y : 0.f);
+    float o[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int s0 = 0; s0 < ns; s0 += 8) {  // eight loads in flight; a piece beyond the last gets weight zero
+      float4 v[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) v[u] = *reinterpret_cast<const float4*>(pc + (size_t)min(s0 + u, ns - 1) * R);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const float f = s0 + u < ns ? __shfl(w, s0 + u) : 0.f;
+        o[0] = fmaf(f, v[u].x, o[0]); o[1] = fmaf(f, v[u].y, o[1]); o[2] = fmaf(f, v[u].z, o[2]); o[3] = fmaf(f, v[u].w, o[3]);
+      }
+    }
+    if (k < R) Tl<T>::st4(xs + tl_off<T>(r, k, R), o);
+  }
+  if (nrow < 16) {  // rows without a position: zeros (their products are dropped, but must be numbers)
+    for (int i = threadIdx.x; i < (16 - nrow) * (R / 4); i += 256) {
+      const float z[4] = {0.f, 0.f, 0.f, 0.f};
+      Tl<T>::st4(xs + tl_off<T>(nrow + i / (R / 4), (i % (R / 4)) * 4, R), z);
     }
   }
   __syncthreads();
@@ -325,10 +459,39 @@ int launch_latent_query(const LatentArgs& a, hipStream_t st) {
   return VUI_OK;
 }
 
-bool latent_mfma_ok(const vui_lm_dims& d) { return false; }
+bool latent_mfma_ok(const vui_lm_dims& d) { return d.rank64 <= 512 && d.rot32 <= 64; }
+
+template <int RK, int RB>
+static int lam_go(const LatentArgs& a, hipStream_t st) {
+  constexpr int lds = 2 * (RK * 2048 + RB * 1024) * 2;
+  if (lds > 60 * 1024) {
+    static bool set = false;
+    if (!set) {
+      HIP_TRY(hipFuncSetAttribute((const void*)latent_attn_mfma_kernel<RK, RB>, hipFuncAttributeMaxDynamicSharedMemorySize, lds));
+      set = true;
+    }
+  }
+  hipLaunchKernelGGL((latent_attn_mfma_kernel<RK, RB>), dim3(a.M, (a.heads + 15) / 16, a.n_splits), dim3(256), lds, st, a);
+  HIP_TRY(hipGetLastError());
+  return VUI_OK;
+}
+template <int RB>
+static int lam_rank(const LatentArgs& a, hipStream_t st) {
+  switch (a.d.rank64 / 64) {
+    case 1: return lam_go<1, RB>(a, st);
+    case 2: return lam_go<2, RB>(a, st);
+    case 3: return lam_go<3, RB>(a, st);
+    case 4: return lam_go<4, RB>(a, st);
+    case 5: return lam_go<5, RB>(a, st);
+    case 6: return lam_go<6, RB>(a, st);
+    case 7: return lam_go<7, RB>(a, st);
+    default: return lam_go<8, RB>(a, st);
+  }
+}
 
 int launch_latent_attn(const LatentArgs& a, hipStream_t st) {
   if (a.n_splits < 1 || a.n_splits > 64 || a.d.rank64 > 256 * LAT_ACC) { vui_set_error("latent attention: rank %d, splits %d out of range", a.d.rank64, a.n_splits); return VUI_EINVAL; }
+  if (a.dtype == VUI_DTYPE_BF16 && latent_mfma_ok(a.d)) return a.d.rot32 == 32 ? lam_rank<1>(a, st) : lam_rank<2>(a, st);
   const dim3 grid(a.M, a.heads, a.n_splits);
   const size_t lds = (size_t)(a.d.rank64 + a.d.rot32) * 4;
   if (a.dtype == VUI_DTYPE_F32) hipLaunchKernelGGL(latent_attn_kernel<float>, grid, dim3(256), lds, st, a);

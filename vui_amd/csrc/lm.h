@@ -98,8 +98,8 @@ struct LatentArgs {
   int own;         // the layer appends latents of its own
   const void *w_uk_t, *w_uv;
   void *c_cache, *kr_cache;
-  // pieces (rows, heads, n_splits, rank64 + 2): max, sum, unnormalised latent average
-  float* part;
+  // pieces (rows, heads, n_splits): unnormalised latent average (rank64), {max, sum}
+  float *part, *part_ml;
   int n_splits;
   const float* gate;
   void* act;

@@ -23,7 +23,7 @@ struct vui_lm_ctx {
   int R16;  // rows of the activation buffers
   float* x; void* xt; float* ssq;
   void *qu, *qr, *qlat;
-  float *craw, *gate, *part;
+  float *craw, *gate, *part, *part_ml;
   void* act;
   float2* upd; void* sg; float2* agg;
   void *kx, *vx;
@@ -54,7 +54,7 @@ static int lm_splits(int M, int heads) {
 static size_t lm_carve(const vui_lm_config* c, const vui_lm_layer* layers, vui_lm_ctx* x, char* base) {
   const size_t e = lm_esz(*c);
   const size_t R = pad(c->max_rows < 16 ? 16 : c->max_rows, 16);
-  size_t qu = 0, qr = 0, ql = 0, cr = 0, ga = 0, pt = 0, ac = 0, up = 0, kx = 0, vx = 0;
+  size_t qu = 0, qr = 0, ql = 0, cr = 0, ga = 0, pt = 0, pm = 0, ac = 0, up = 0, kx = 0, vx = 0;
   vui_lm_dims d;
   memset(&d, 0, sizeof(d));
   auto mx = [](size_t& a, size_t b) { if (b > a) a = b; };
@@ -68,7 +68,7 @@ static size_t lm_carve(const vui_lm_config* c, const vui_lm_layer* layers, vui_l
     mx(cr, R * d.rank16); mx(ga, R * d.heads16);
     size_t rows = R;  // rows x splits of attention pieces
     for (int M = 1; M <= (int)R && M <= 256; ++M) mx(rows, (size_t)M * lm_splits(M, L.heads));
-    mx(pt, rows * H * (d.rank64 + 2));
+    mx(pt, rows * H * d.rank64); mx(pm, rows * H * 2);
     if (lm_expands(*c, d)) { mx(kx, H * d.s64 * d.dim64); mx(vx, H * d.s64 * d.vdim16); }
   }
   size_t off = 0;
@@ -83,6 +83,7 @@ static size_t lm_carve(const vui_lm_config* c, const vui_lm_layer* layers, vui_l
   TAKE(craw, float*, cr * 4);
   TAKE(gate, float*, ga * 4);
   TAKE(part, float*, pt * 4);
+  TAKE(part_ml, float*, pm * 4);
   TAKE(act, void*, ac * e);
   TAKE(upd, float2*, R * up * 8);
   TAKE(sg, void*, R * up * e);
@@ -228,7 +229,7 @@ static int lm_attention(vui_lm_ctx* x, int l, int M, const LmRows& rows, LmGemm&
   a.qlat = x->qlat; a.qlat_z = (size_t)x->R16 * d.rank64;
   a.craw = x->craw; a.latent_norm = L.latent_norm; a.eps = c.norm_eps; a.own = own;
   a.w_uk_t = L.w_uk_t; a.w_uv = L.w_uv; a.c_cache = L.c_cache; a.kr_cache = L.kr_cache;
-  a.part = x->part; a.gate = x->gate; a.act = x->act;
+  a.part = x->part; a.part_ml = x->part_ml; a.gate = x->gate; a.act = x->act;
   if (rows.seq && M >= x->expand_from && lm_expands(c, d)) {
     if (own && (rc = launch_latent_append(a, st))) return rc;
     LmGemm k;

@@ -109,3 +109,67 @@ def synthetic_codec_state_dict(cfg, seed: int = 0) -> dict[str, Tensor]:
             t = r / math.sqrt(shape[-1])
         sd[k] = t.contiguous()
     return sd
+
+
+def token_lm_config(width: int, heads: int, ff: int, dim: int, rot_dim: int, vdim: int, kv_rank: int, n_layers: int,
+                    vocab: int = 8192, rnn_width: int = 0) -> dict:
+    """A Sakupel configuration whose layers repeat the pattern: attention with latents of its own, attention on the same
+    latents, minGRU, attention with latents of its own."""
+    layers = []
+    own = 0
+    for i in range(n_layers):
+        mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+        if i % 4 == 2:
+            layers.append({"type": "mingru", "mixer": {"width": rnn_width or width}, "mlp": mlp})
+            continue
+        mx = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank,
+              "scale": (dim + rot_dim) ** -0.5, "rot": {"dims": rot_dim, "base": 10000.0}}
+        if i % 4 == 1:
+            mx["kv_from"] = own
+        else:
+            own = i
+        layers.append({"type": "latent_attention", "mixer": mx, "mlp": mlp})
+    return {"architecture": "Sakupel", "width": width, "vocab": vocab, "norm": {"eps": 1e-5}, "layers": layers}
+
+
+def token_lm_state_dict(cfg: dict, seed: int = 0, device="cpu") -> dict[str, Tensor]:
+    """Random bf16 weights N(0, 1 / fan_in) of a token model's configuration, norm weights 1, biases 0."""
+    g = torch.Generator(device=device).manual_seed(seed)
+    W = cfg["width"]
+    sd: dict[str, Tensor] = {}
+
+    def mat(name: str, n: int, k: int) -> None:
+        sd[name] = (torch.randn(n, k, generator=g, device=device) * k ** -0.5).to(torch.bfloat16)
+
+    def ones(name: str, *shape: int) -> None:
+        sd[name] = torch.ones(shape, dtype=torch.bfloat16, device=device)
+
+    mat("embed", cfg["vocab"], W)
+    for i, layer in enumerate(cfg["layers"]):
+        p, mx = f"l{i}.", layer["mixer"]
+        ones(p + "norm1")
+        if layer["type"] == "latent_attention":
+            H, r = mx["heads"], mx["kv_rank"]
+            mat(p + "mix.q", H * (mx["dim"] + mx["rot_dim"]), W)
+            if mx.get("kv_from") is None:
+                mat(p + "mix.dkv", r + mx["rot_dim"], W)
+                ones(p + "mix.dkv.norm", r)
+            mat(p + "mix.uk", H * mx["dim"], r)
+            mat(p + "mix.uv", H * mx["vdim"], r)
+            mat(p + "mix.g", H, W)
+            mat(p + "mix.o", W, H * mx["vdim"])
+        else:
+            n = mx["width"]
+            for k in ("z", "x", "g"):
+                mat(p + "mix." + k, n, W)
+            for k in ("z.b", "x.b"):
+                sd[p + "mix." + k] = torch.zeros(n, dtype=torch.bfloat16, device=device)
+            mat(p + "mix.o", W, n)
+        if layer["mlp"] is not None:
+            f = layer["mlp"]["ff"]
+            mat(p + "mlp.gate", f, W)
+            mat(p + "mlp.up", f, W)
+            mat(p + "mlp.down", W, f)
+    ones("final.norm")
+    mat("head", cfg["vocab"], W)
+    return sd
