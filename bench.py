@@ -564,7 +564,7 @@ def lm_lines(sizes=None, batches=(1, 4, 16), prompts=(512, 2048), L=1024, which=
         torch.cuda.synchronize()
         return e0.elapsed_time(e1) * 1e3 / n
 
-    S = 2304
+    S = max(2304, L + 256, max(prompts, default=0) + 16)
     for name, W, H, F, dim, rot, vdim, rank, nl in LM_SIZES:
         if sizes and name not in sizes:
             continue
@@ -608,7 +608,7 @@ def lm_lines(sizes=None, batches=(1, 4, 16), prompts=(512, 2048), L=1024, which=
                 by = (wl + W * 2048) * 2 + B * L * nl * 4 * W
                 vui[f"decode_b{B}"] = {"us": round(us, 1), "tokens_per_s": round(B * 1e6 / us), "GBs": round(by / us / 1e3, 1), "hbm_frac": round(by / us / 1e3 / HBM_PEAK_GBS, 4)}
                 vui["forms"][f"b{B}"] = "one launch" if (vm._native.fused(-1) if B == 1 else vm._native.bb_batch()) else "kernel sequence"
-                if B == batches[0]:
+                if B == batches[0] and prompts:
                     emb = (torch.randn(1, max(prompts), W, device="cuda") * 0.1).to(torch.bfloat16)
                     for T in prompts:
                         def pre():
@@ -863,6 +863,7 @@ def main():
     ap.add_argument("--lm-which", default="both", choices=["both", "lm", "vui"], help="one side of the --lm lines (for profiles)")
     ap.add_argument("--lm-batch", type=int, nargs="*", default=[1, 4, 16], help="rows of the --lm decode steps")
     ap.add_argument("--lm-prompt", type=int, nargs="*", default=[512, 2048], help="prompt lengths of the --lm lines")
+    ap.add_argument("--lm-length", type=int, default=1024, help="cache length of the --lm decode steps")
     ap.add_argument("--phase-clock", action="store_true",
                     help="print the phase stamps of one workgroup of the batch-1 frame kernel (with --int8: int8 weights)")
     ap.add_argument("--bb-phase-clock", type=int, default=0, metavar="ROWS",
@@ -876,7 +877,7 @@ def main():
               "run with --gpus 1", file=sys.stderr)
         sys.exit(2)
     if args.lm is not None:
-        for ln in lm_lines(args.lm, args.lm_batch, args.lm_prompt, which=args.lm_which):
+        for ln in lm_lines(args.lm, args.lm_batch, args.lm_prompt, L=args.lm_length, which=args.lm_which):
             print(json.dumps(ln), flush=True)
         return
     if args.phase_clock:

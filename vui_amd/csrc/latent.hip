@@ -73,10 +73,11 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const LatentArgs p) {
   Tl<T>::st4((T*)p.qlat + h * p.qlat_z + tl_off<T>(m, nb * 16 + 4 * (lane >> 4), p.d.rank64), v);
 }
 
-// keys [lo, hi) of split sp of a row that sees len keys
+// A row that sees len keys is cut into pieces of this many (whole 32-key tiles, at least two), at most ns of them.
+__device__ __forceinline__ int latent_chunk(int len, int ns) { return max(((len + ns - 1) / ns + 31) & ~31, 64); }
+// keys [lo, hi) of piece sp
 __device__ __forceinline__ void latent_range(int len, int ns, int sp, int& lo, int& hi) {
-  int chunk = (len + ns - 1) / ns;
-  chunk = (chunk + 31) & ~31;
+  const int chunk = latent_chunk(len, ns);
   lo = min(sp * chunk, len);
   hi = min(lo + chunk, len);
 }
@@ -96,6 +97,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs p) {
   const int len = min(max(lm_pos(p.rows, m, slot) + 1, 1), p.rows.S);
   int lo, hi;
   latent_range(len, p.n_splits, sp, lo, hi);
+  if (lo >= hi) return;  // no such piece: latent_value_kernel does not look for it
   for (int k = tid; k < R + RR; k += 256)
     lq[k] = k < R ? (k < p.d.rank16 ? El<T>::ld((const T*)p.qlat + h * p.qlat_z + tl_off<T>(m, k, R)) : 0.f)
                   : (k - R < p.d.rot16 ? El<T>::ld((const T*)p.qr + h * p.qr_z + tl_off<T, 32>(m, k - R, RR)) : 0.f);
@@ -161,8 +163,6 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs p) {
 // RK = rank64 / 64, RB = rot32 / 32.
 template <int RK, int RB>
 __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const LatentArgs p) {
-  constexpr int NC = 2 * RK + RB;         // 32-column chunks of a key row
-  constexpr int NQ = (NC + 1) / 2;        // chunks per wave
   constexpr int CT = RK * 2048, RT = RB * 1024;  // elements of the staged tiles (32 keys)
   extern __shared__ __align__(16) bf16_t tile[];  // 2 x (CT + RT)
   __shared__ __align__(16) float sco[4][64 * 4];
@@ -174,51 +174,48 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const LatentArgs 
   const int len = min(max(lm_pos(p.rows, m, slot) + 1, 1), p.rows.S);
   int lo, hi;
   latent_range(len, p.n_splits, sp, lo, hi);
-  const uint4* cc = reinterpret_cast<const uint4*>((const bf16_t*)p.c_cache + (size_t)slot * p.d.s64 * (RK * 64));
-  const uint4* kc = reinterpret_cast<const uint4*>((const bf16_t*)p.kr_cache + (size_t)slot * p.d.s64 * (RB * 32));
+  const tl_u32x4* cc = reinterpret_cast<const tl_u32x4*>((const bf16_t*)p.c_cache + (size_t)slot * p.d.s64 * (RK * 64));
+  const tl_u32x4* kc = reinterpret_cast<const tl_u32x4*>((const bf16_t*)p.kr_cache + (size_t)slot * p.d.s64 * (RB * 32));
+  if (lo >= hi) return;  // no such piece
   // 32 keys are one contiguous run of either cache
-  uint4 rc[RK], rr = make_uint4(0, 0, 0, 0);
-  auto fetch = [&](int j0) {
-#pragma unroll
-    for (int i = 0; i < RK; ++i) rc[i] = cc[(size_t)(j0 >> 5) * (CT / 8) + tid + 256 * i];
-    rr = kc[(size_t)(j0 >> 5) * (RT / 8) + min(tid, RT / 8 - 1)];
-  };
-  auto stage = [&](bf16_t* dst) {
-    uint4* d = reinterpret_cast<uint4*>(dst);
-#pragma unroll
-    for (int i = 0; i < RK; ++i) d[tid + 256 * i] = rc[i];
-    if (tid < RT / 8) d[CT / 8 + tid] = rr;
-  };
-  if (lo < hi) fetch(lo);
-  uint4 qf[NQ];
-#pragma unroll
-  for (int i = 0; i < NQ; ++i) {
-    const int c = min(2 * i + half, NC - 1);
-    const bf16_t* src = c < 2 * RK
-        ? (const bf16_t*)p.qlat + hq * p.qlat_z + ((size_t)(m >> 4) * RK + (c >> 1)) * 1024 + (c & 1) * 512 + ((m & 15) + 16 * kg) * 8
-        : (const bf16_t*)p.qr + hq * p.qr_z + ((size_t)(m >> 4) * RB + (c - 2 * RK)) * 512 + ((m & 15) + 16 * kg) * 8;
-    qf[i] = *reinterpret_cast<const uint4*>(src);
+  tl_u32x4 rc[RK], rr;
+#define LAT_FETCH(j)                                                                            \
+  {                                                                                             \
+    const size_t jt = (size_t)((j) >> 5);                                                       \
+    _Pragma("unroll") for (int i = 0; i < RK; ++i) rc[i] = cc[jt * (CT / 8) + tid + 256 * i];   \
+    rr = kc[jt * (RT / 8) + min(tid, RT / 8 - 1)];                                              \
   }
+#define LAT_STAGE(dst)                                                                          \
+  {                                                                                             \
+    tl_u32x4* sd = reinterpret_cast<tl_u32x4*>(dst);                                                  \
+    _Pragma("unroll") for (int i = 0; i < RK; ++i) sd[tid + 256 * i] = rc[i];                   \
+    if (tid < RT / 8) sd[CT / 8 + tid] = rr;                                                    \
+  }
+  LAT_FETCH(lo);
+  // this wave's columns: piece `half` of every latent block, and a block of the rotated part (one wave pair without, RB = 1)
+  const bool rot = RB == 2 || half == 0;
+  uint4 qf[RK + 1];
+  const int qrow = ((m & 15) + 16 * kg) * 8;
+#pragma unroll
+  for (int i = 0; i < RK; ++i)
+    qf[i] = *reinterpret_cast<const uint4*>((const bf16_t*)p.qlat + hq * p.qlat_z + ((size_t)(m >> 4) * RK + i) * 1024 + half * 512 + qrow);
+  qf[RK] = *reinterpret_cast<const uint4*>((const bf16_t*)p.qr + hq * p.qr_z + ((size_t)(m >> 4) * RB + (RB == 2 ? half : 0)) * 512 + qrow);
   tl_f32x4 acc[RK];
 #pragma unroll
   for (int i = 0; i < RK; ++i) acc[i] = tl_f32x4{0.f, 0.f, 0.f, 0.f};
   float m_run = -INFINITY, l_run = 0.f;
-  if (lo < hi) stage(tile);
+  LAT_STAGE(tile);
   __syncthreads();
   int buf = 0;
   for (int j0 = lo; j0 < hi; j0 += 32) {
     const bf16_t* cur = tile + buf * (CT + RT);
     const bool more = j0 + 32 < hi;
-    if (more) fetch(j0 + 32);
+    LAT_FETCH(more ? j0 + 32 : j0);
     tl_f32x4 s = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int i = 0; i < NQ; ++i) {
-      const int c = 2 * i + half;
-      if (c < NC) {  // uniform over the wave
-        const bf16_t* a = c < 2 * RK ? cur + (t * RK + (c >> 1)) * 1024 + (c & 1) * 512 : cur + CT + (t * RB + (c - 2 * RK)) * 512;
-        s = Tl<bf16_t>::mma(*reinterpret_cast<const uint4*>(a + lane * 8), qf[i], s);
-      }
-    }
+    for (int i = 0; i < RK; ++i) s = Tl<bf16_t>::mma(*reinterpret_cast<const uint4*>(cur + (t * RK + i) * 1024 + half * 512 + lane * 8), qf[i], s);
+    if (rot)  // uniform over the wave
+      s = Tl<bf16_t>::mma(*reinterpret_cast<const uint4*>(cur + CT + (t * RB + (RB == 2 ? half : 0)) * 512 + lane * 8), qf[RK], s);
     *reinterpret_cast<tl_f32x4*>(&sco[half * 2 + t][lane * 4]) = s;
     __syncthreads();
     // keys j0 + 16 u + 4 kg + r of this lane's head
@@ -260,7 +257,7 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const LatentArgs 
       acc[i] = Tl<bf16_t>::mma(v, hi4, acc[i]);
       acc[i] = Tl<bf16_t>::mma(v, lo4, acc[i]);
     }
-    if (more) stage(tile + (buf ^ 1) * (CT + RT));
+    if (more) LAT_STAGE(tile + (buf ^ 1) * (CT + RT));
     __syncthreads();
     buf ^= 1;
   }
@@ -273,63 +270,74 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const LatentArgs 
     *reinterpret_cast<tl_f32x4*>(p.part + piece * (RK * 64) + i * 64 + wave * 16 + 4 * kg) = acc[i];
 }
 
-// ---- merge of the pieces, value expansion through W_uv[h], head gate: 16 rows x up to 64 value dims of one head ----
+// ---- merge of the pieces, value expansion through W_uv[h], head gate: up to 16 rows x 128 value dims of one head ----
 template <typename T>
-__global__ __launch_bounds__(256) void latent_value_kernel(const LatentArgs p) {
+__global__ __launch_bounds__(512) void latent_value_kernel(const LatentArgs p, int rpw) {
   extern __shared__ __align__(16) unsigned char lv_raw[];
   T* xs = (T*)lv_raw;  // 16 x rank64, tiled
-  constexpr int EP = Tl<T>::EP, P = 16 / EP;
+  constexpr int EP = Tl<T>::EP, P = 16 / EP, PRE = sizeof(T) == 2 ? 8 : 4;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
-  const int h = blockIdx.x, mt = blockIdx.z, R = p.d.rank64, ns = p.n_splits;
-  const int nrow = min(16, p.M - mt * 16), ncol = (R + 255) / 256;
-  for (int it = wave; it < nrow * ncol; it += 4) {  // a wave merges 256 columns of a row
-    const int r = it / ncol, k = (it - r * ncol) * 256 + 4 * lane;
-    const size_t piece = ((size_t)(mt * 16 + r) * p.heads + h) * ns;
-    const float2 ml = *reinterpret_cast<const float2*>(p.part_ml + 2 * (piece + min(lane, ns - 1)));
-    const float* pc = p.part + piece * R + min(k, R - 4);
-    const float ms = lane < ns ? ml.x : -INFINITY;
-    const float M = wave_max(ms);
-    float w = ms == -INFINITY ? 0.f : expf(ms - M);
-    w /= wave_sum(lane < ns ? w * ml.y : 0.f);
-    float o[4] = {0.f, 0.f, 0.f, 0.f};
-    for (int s0 = 0; s0 < ns; s0 += 8) {  // eight loads in flight; a piece beyond the last gets weight zero
-      float4 v[8];
+  const int h = blockIdx.x, m0 = blockIdx.z * rpw, R = p.d.rank64, ns = p.n_splits, nk = R >> 6;
+  const int nb = blockIdx.y * 8 + wave, nvb = p.d.vdim16 >> 4;
+  const int nrow = min(rpw, p.M - m0);
+  const float gate = p.gate[(size_t)min(m0 + (lane & 15), p.M - 1) * p.d.heads16 + h];
+  // the first weights are requested ahead of the merge
+  const T* wv = (const T*)p.w_uv + ((size_t)h * nvb + min(nb, nvb - 1)) * nk * 1024 + lane * EP;
+  uint4 wp[PRE][P];
 #pragma unroll
-      for (int u = 0; u < 8; ++u) v[u] = *reinterpret_cast<const float4*>(pc + (size_t)min(s0 + u, ns - 1) * R);
+  for (int k = 0; k < PRE; ++k)
 #pragma unroll
-      for (int u = 0; u < 8; ++u) {
-        const float f = s0 + u < ns ? __shfl(w, s0 + u) : 0.f;
-        o[0] = fmaf(f, v[u].x, o[0]); o[1] = fmaf(f, v[u].y, o[1]); o[2] = fmaf(f, v[u].z, o[2]); o[3] = fmaf(f, v[u].w, o[3]);
-      }
+    for (int i = 0; i < P; ++i) wp[k][i] = *reinterpret_cast<const uint4*>(wv + (size_t)min(k, nk - 1) * 1024 + 64 * EP * i);
+  for (int it = wave; it < nrow * nk; it += 8) {  // a wave merges 64 columns of a row
+    const int r = it / nk, k = (it - r * nk) * 64 + lane;
+    const int m = m0 + r, slot = lm_slot(p.rows, m);
+    const int len = min(max(lm_pos(p.rows, m, slot) + 1, 1), p.rows.S);
+    const int chunk = latent_chunk(len, ns), np = (len + chunk - 1) / chunk;  // pieces that exist
+    const size_t piece = ((size_t)m * p.heads + h) * ns;
+    const float2 ml = *reinterpret_cast<const float2*>(p.part_ml + 2 * (piece + min(lane, np - 1)));
+    const float* pc = p.part + piece * R + k;
+    float v[16];  // sixteen loads in flight; a piece beyond the last gets weight zero
+#pragma unroll
+    for (int u = 0; u < 16; ++u) v[u] = pc[(size_t)min(u, np - 1) * R];
+    const float M = wave_max(lane < np ? ml.x : -INFINITY);
+    float w = lane < np ? expf(ml.x - M) : 0.f;
+    w /= wave_sum(w * ml.y);
+    float o = 0.f;
+    for (int s0 = 0;;) {
+#pragma unroll
+      for (int u = 0; u < 16; ++u) o = fmaf(lane_f(w, min(s0 + u, 63)), s0 + u < np ? v[u] : 0.f, o);
+      s0 += 16;
+      if (s0 >= np) break;
+#pragma unroll
+      for (int u = 0; u < 16; ++u) v[u] = pc[(size_t)min(s0 + u, np - 1) * R];
     }
-    if (k < R) Tl<T>::st4(xs + tl_off<T>(r, k, R), o);
+    El<T>::st(xs + tl_off<T>(r, k, R), o);
   }
-  if (nrow < 16) {  // rows without a position: zeros (their products are dropped, but must be numbers)
-    for (int i = threadIdx.x; i < (16 - nrow) * (R / 4); i += 256) {
-      const float z[4] = {0.f, 0.f, 0.f, 0.f};
-      Tl<T>::st4(xs + tl_off<T>(nrow + i / (R / 4), (i % (R / 4)) * 4, R), z);
-    }
+  // rows without a position: their products are dropped, but must be numbers
+  for (int i = threadIdx.x; i < (16 - nrow) * (R / 4); i += 512) {
+    const float z[4] = {0.f, 0.f, 0.f, 0.f};
+    Tl<T>::st4(xs + tl_off<T>(nrow + i / (R / 4), (i % (R / 4)) * 4, R), z);
   }
   __syncthreads();
-  const int nb = blockIdx.y * 4 + wave;
-  if (nb >= p.d.vdim16 >> 4) return;
-  const int nk = R >> 6;
-  const T* wv = (const T*)p.w_uv + ((size_t)h * (p.d.vdim16 >> 4) + nb) * nk * 1024 + lane * EP;
+  if (nb >= nvb) return;
   tl_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-  for (int k = 0; k < nk; ++k) {
-    uint4 a[P], b[P];
+  auto step = [&](int k, const uint4* a) {
 #pragma unroll
-    for (int i = 0; i < P; ++i) {
-      a[i] = *reinterpret_cast<const uint4*>(wv + (size_t)k * 1024 + 64 * EP * i);
-      b[i] = *reinterpret_cast<const uint4*>(xs + (size_t)k * 1024 + 64 * EP * i + lane * EP);
-    }
+    for (int i = 0; i < P; ++i)
+      acc = Tl<T>::mma(a[i], *reinterpret_cast<const uint4*>(xs + (size_t)k * 1024 + 64 * EP * i + lane * EP), acc);
+  };
 #pragma unroll
-    for (int i = 0; i < P; ++i) acc = Tl<T>::mma(a[i], b[i], acc);
+  for (int k = 0; k < PRE; ++k)
+    if (k < nk) step(k, wp[k]);
+  for (int k = PRE; k < nk; ++k) {
+    uint4 a[P];
+#pragma unroll
+    for (int i = 0; i < P; ++i) a[i] = *reinterpret_cast<const uint4*>(wv + (size_t)k * 1024 + 64 * EP * i);
+    step(k, a);
   }
-  const int m = mt * 16 + (lane & 15);
-  if (m >= p.M) return;
-  const float g = p.gate[(size_t)m * p.d.heads16 + h];
-  const float v[4] = {acc[0] * g, acc[1] * g, acc[2] * g, acc[3] * g};
+  const int m = m0 + (lane & 15);
+  if ((lane & 15) >= nrow) return;
+  const float v[4] = {acc[0] * gate, acc[1] * gate, acc[2] * gate, acc[3] * gate};
   Tl<T>::st4((T*)p.act + tl_off<T>(m, h * p.d.vdim16 + nb * 16 + 4 * (lane >> 4), p.d.out_k), v);
 }
 
@@ -501,15 +509,18 @@ int launch_latent_attn(const LatentArgs& a, hipStream_t st) {
 }
 
 int launch_latent_value(const LatentArgs& a, hipStream_t st) {
-  const dim3 grid(a.heads, (a.d.vdim16 / 16 + 3) / 4, (a.M + 15) / 16);
+  // rows per workgroup: all 16 of a tile only when there are enough heads and rows to fill the chip without
+  int rpw = 1;
+  while (rpw < 16 && a.M * a.heads > 192 * rpw) rpw *= 2;
+  const dim3 grid(a.heads, (a.d.vdim16 / 16 + 7) / 8, (a.M + rpw - 1) / rpw);
   const bool f32 = a.dtype == VUI_DTYPE_F32;
   const size_t lds = (size_t)16 * a.d.rank64 * (f32 ? 4 : 2);
   if (lds > 64 * 1024) {
     HIP_TRY(hipFuncSetAttribute(f32 ? (const void*)latent_value_kernel<float> : (const void*)latent_value_kernel<bf16_t>,
                                 hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
   }
-  if (f32) hipLaunchKernelGGL(latent_value_kernel<float>, grid, dim3(256), lds, st, a);
-  else hipLaunchKernelGGL(latent_value_kernel<bf16_t>, grid, dim3(256), lds, st, a);
+  if (f32) hipLaunchKernelGGL(latent_value_kernel<float>, grid, dim3(512), lds, st, a, rpw);
+  else hipLaunchKernelGGL(latent_value_kernel<bf16_t>, grid, dim3(512), lds, st, a, rpw);
   HIP_TRY(hipGetLastError());
   return VUI_OK;
 }

@@ -11,7 +11,7 @@
 #include "lm.h"
 
 #define LM_EXPAND_FROM 64   // positions of one call from which keys and values are expanded per head
-#define LM_MAX_SPLITS 16
+#define LM_MAX_SPLITS 64   // latent_value_kernel keeps one piece per lane
 
 static int pad(int v, int a) { return (v + a - 1) / a * a; }
 
@@ -45,9 +45,10 @@ static size_t lm_esz(const vui_lm_config& c) { return c.dtype == VUI_DTYPE_F32 ?
 
 static bool lm_expands(const vui_lm_config& c, const vui_lm_dims& d) { return c.dtype == VUI_DTYPE_BF16 && latent_expand_ok(d); }
 
-// n_splits of attention in the latent space: about one workgroup per compute unit
-static int lm_splits(int M, int heads) {
-  const int t = 256 / (M * ((heads + 15) / 16));
+// n_splits of attention in the latent space: as many workgroups as stay resident beside each other (LDS holds two
+// staged tiles of 32 latents per workgroup)
+static int lm_splits(int M, int heads, int rank64) {
+  const int t = (rank64 <= 256 ? 1024 : 512) / (M * ((heads + 15) / 16));
   return t < 1 ? 1 : (t > LM_MAX_SPLITS ? LM_MAX_SPLITS : t);
 }
 
@@ -67,7 +68,7 @@ static size_t lm_carve(const vui_lm_config* c, const vui_lm_layer* layers, vui_l
     mx(qu, H * R * d.dim64); mx(qr, H * R * d.rot32); mx(ql, H * R * d.rank64);
     mx(cr, R * d.rank16); mx(ga, R * d.heads16);
     size_t rows = R;  // rows x splits of attention pieces
-    for (int M = 1; M <= (int)R && M <= 256; ++M) mx(rows, (size_t)M * lm_splits(M, L.heads));
+    for (int M = 1; M <= (int)R && M <= 1024; ++M) mx(rows, (size_t)M * lm_splits(M, L.heads, d.rank64));
     mx(pt, rows * H * d.rank64); mx(pm, rows * H * 2);
     if (lm_expands(*c, d)) { mx(kx, H * d.s64 * d.dim64); mx(vx, H * d.s64 * d.vdim16); }
   }
@@ -243,7 +244,7 @@ static int lm_attention(vui_lm_ctx* x, int l, int M, const LmRows& rows, LmGemm&
     a.kx = x->kx; a.vx = x->vx; a.kx_z = (size_t)d.s64 * d.dim64; a.vx_z = (size_t)d.s64 * d.vdim16;
     return launch_latent_prefill_attn(a, st);
   }
-  a.n_splits = lm_splits(M, L.heads);
+  a.n_splits = lm_splits(M, L.heads, d.rank64);
   if ((rc = launch_latent_query(a, st))) return rc;
   if ((rc = launch_latent_attn(a, st))) return rc;
   return launch_latent_value(a, st);

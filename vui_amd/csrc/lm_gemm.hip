@@ -55,34 +55,77 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
       const int r = min(max(p.rowmap[min(m0 + 16 * j + l16, p.M - 1)], 0), p.x_rows - 1);
       xr[j] = (const T*)p.X + (size_t)(r >> 4) * nsteps * 1024 + ((r & 15) + 16 * kg) * EP;
     } else {
-      xr[j] = (const T*)p.X + (size_t)min((m0 >> 4) + j, MBL - 1) * nsteps * 1024 + lane * EP;
+      // few rows: lanes without a row re-read the last one instead of fetching a block that is mostly padding
+      const int l = MB == 1 && !ROWS_FIRST ? min(l16, p.M - 1 - m0) + 16 * kg : lane;
+      xr[j] = (const T*)p.X + (size_t)min((m0 >> 4) + j, MBL - 1) * nsteps * 1024 + l * EP;
     }
   }
 #pragma unroll
   for (int i = 0; i < NB; ++i)
     wr[i] = (const T*)p.W + blockIdx.z * p.wz + (size_t)min(nb0 + i, NBL - 1) * nsteps * 1024 + lane * EP;
 
+  // What the scale and the epilogue of this wave's first unit will need is requested now, ahead of the operands:
+  // fetched where it is used, it would be a chain of dependent loads behind the last product.
+  // Scale: TPR neighbouring threads add up one row's sums of squares, in a fixed order.
+  constexpr int TPR = WAVES * 64 / (MB * 16) > 64 ? 64 : WAVES * 64 / (MB * 16), NSQ = 4;
+  const int sq_r = tid / TPR, sq_q = tid % TPR;
+  int sq_m = 0;
+  float sq[NSQ], norm = 0.f;
+  if (SCALED) {
+    sq_m = min(m0 + min(sq_r, MB * 16 - 1), p.M - 1);
+    if (EPI == LM_LOGITS && p.rowmap) sq_m = min(max(p.rowmap[sq_m], 0), p.x_rows - 1);
+#pragma unroll
+    for (int i = 0; i < NSQ; ++i) sq[i] = p.ssq[(size_t)sq_m * p.np + min(sq_q + TPR * i, p.np - 1)];
+    norm = p.norm[0];
+  }
+  constexpr bool PRE = MB == 1 && (EPI == LM_IN_ATTN || EPI == LM_IN_GRU_STEP || EPI == LM_OUT);
+  const int pm = min(m0 + l16, p.M - 1), pb = min(nb0 + min(wave, NB - 1), NBL - 1);  // row and block of unit `wave`
+  int e_slot = 0, e_pos = 0;
+  float4 e_a = make_float4(0.f, 0.f, 0.f, 0.f), e_b = e_a, e_c = e_a;
+  if (PRE && EPI != LM_OUT) {
+    e_slot = lm_slot(p.rows, pm);
+    e_pos = lm_pos(p.rows, pm, e_slot);
+  }
+  if (PRE && EPI == LM_OUT) e_a = *reinterpret_cast<const float4*>(p.x + (size_t)pm * p.d.w64 + pb * 16 + 4 * kg);
+  if (PRE && EPI == LM_IN_GRU_STEP && nb0 < p.mix_blocks) {
+    const int ch = (nb0 / 3) * 16 + 4 * kg;
+    e_a = *reinterpret_cast<const float4*>(p.state + (size_t)e_slot * p.d.gru16 + ch);
+    e_b = *reinterpret_cast<const float4*>(p.bz + ch);
+    e_c = *reinterpret_cast<const float4*>(p.bx + ch);
+  }
+
   tl_f32x4 acc[NB][MB];
 #pragma unroll
   for (int i = 0; i < NB; ++i)
 #pragma unroll
     for (int j = 0; j < MB; ++j) acc[i][j] = tl_f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int s = s0; s < s1; ++s) {
-    uint4 xa[MB][P], wa[NB][P];
+  // U steps' loads go out together (a step beyond the wave's last re-reads that one and is not multiplied)
+  constexpr int U = WAVES >= 8 && sizeof(T) == 2 ? 4 : 1;
+  for (int s = s0; s < s1; s += U) {
+    uint4 xa[U][MB][P], wa[U][NB][P];
 #pragma unroll
-    for (int h = 0; h < P; ++h) {
+    for (int u = 0; u < U; ++u) {
+      const size_t o = (size_t)min(s + u, s1 - 1) * 1024;
 #pragma unroll
-      for (int i = 0; i < NB; ++i) wa[i][h] = *reinterpret_cast<const uint4*>(wr[i] + (size_t)s * 1024 + 64 * EP * h);
+      for (int h = 0; h < P; ++h) {
 #pragma unroll
-      for (int j = 0; j < MB; ++j) xa[j][h] = *reinterpret_cast<const uint4*>(xr[j] + (size_t)s * 1024 + 64 * EP * h);
+        for (int i = 0; i < NB; ++i) wa[u][i][h] = *reinterpret_cast<const uint4*>(wr[i] + o + 64 * EP * h);
+#pragma unroll
+        for (int j = 0; j < MB; ++j) xa[u][j][h] = *reinterpret_cast<const uint4*>(xr[j] + o + 64 * EP * h);
+      }
     }
+    __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-    for (int h = 0; h < P; ++h)
+    for (int u = 0; u < U; ++u) {
+      if (s + u >= s1) break;  // uniform
 #pragma unroll
-      for (int i = 0; i < NB; ++i)
+      for (int h = 0; h < P; ++h)
 #pragma unroll
-        for (int j = 0; j < MB; ++j)
-          acc[i][j] = ROWS_FIRST ? Tl<T>::mma(xa[j][h], wa[i][h], acc[i][j]) : Tl<T>::mma(wa[i][h], xa[j][h], acc[i][j]);
+        for (int i = 0; i < NB; ++i)
+#pragma unroll
+          for (int j = 0; j < MB; ++j)
+            acc[i][j] = ROWS_FIRST ? Tl<T>::mma(xa[u][j][h], wa[u][i][h], acc[i][j]) : Tl<T>::mma(wa[u][i][h], xa[u][j][h], acc[i][j]);
+    }
   }
 #pragma unroll
   for (int i = 0; i < NB; ++i)
@@ -90,18 +133,13 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
     for (int j = 0; j < MB; ++j)
       *reinterpret_cast<tl_f32x4*>(&part[wave * TILE + ((i * MB + j) * 64 + lane) * 4]) = acc[i][j];
   if (SCALED) {
-    // TPR neighbouring threads add up one row's sums of squares, in a fixed order
-    constexpr int TPR = WAVES * 64 / (MB * 16) > 64 ? 64 : WAVES * 64 / (MB * 16);
-    const int r = tid / TPR, q = tid % TPR;
-    float s = 0.f;
-    if (r < MB * 16) {
-      int m = min(m0 + r, p.M - 1);
-      if (EPI == LM_LOGITS && p.rowmap) m = min(max(p.rowmap[m], 0), p.x_rows - 1);
-      for (int i = q; i < p.np; i += TPR) s += p.ssq[(size_t)m * p.np + i];
-    }
+    float t = 0.f;
 #pragma unroll
-    for (int o = TPR / 2; o >= 1; o >>= 1) s += __shfl_xor(s, o);
-    if (r < MB * 16 && q == 0) srow[r] = p.norm[0] / sqrtf(s / (float)p.width + p.eps);
+    for (int i = 0; i < NSQ; ++i) t += sq_q + TPR * i < p.np ? sq[i] : 0.f;
+    for (int i = sq_q + TPR * NSQ; i < p.np; i += TPR) t += p.ssq[(size_t)sq_m * p.np + i];
+#pragma unroll
+    for (int o = TPR / 2; o >= 1; o >>= 1) t += __shfl_xor(t, o);
+    if (sq_r < MB * 16 && sq_q == 0) srow[sq_r] = norm / sqrtf(t / (float)p.width + p.eps);
   }
   __syncthreads();
 
@@ -131,7 +169,7 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
       gather(NB > 2 ? 2 : 0, gv);
       const int ch = (nb / 3) * 16 + 4 * kg;  // blocks come in threes: update gate, candidate, output gate
       if (!live) continue;
-      const float4 b0 = *reinterpret_cast<const float4*>(p.bz + ch), b1 = *reinterpret_cast<const float4*>(p.bx + ch);
+      const float4 b0 = PRE ? e_b : *reinterpret_cast<const float4*>(p.bz + ch), b1 = PRE ? e_c : *reinterpret_cast<const float4*>(p.bx + ch);
       const float zb[4] = {b0.x, b0.y, b0.z, b0.w}, xb[4] = {b1.x, b1.y, b1.z, b1.w};
       float keep[4], in[4], sg[4];
 #pragma unroll
@@ -143,9 +181,8 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
         sg[r] = gv[r] * lm_sigmoid(gv[r]);
       }
       if (EPI == LM_IN_GRU_STEP) {
-        const int slot = lm_slot(p.rows, m), pos = lm_pos(p.rows, m, slot);
-        float4* sp = reinterpret_cast<float4*>(p.state + (size_t)slot * p.d.gru16 + ch);
-        const float4 old = pos > 0 ? *sp : make_float4(0.f, 0.f, 0.f, 0.f);
+        float4* sp = reinterpret_cast<float4*>(p.state + (size_t)e_slot * p.d.gru16 + ch);
+        const float4 old = e_pos > 0 ? e_a : make_float4(0.f, 0.f, 0.f, 0.f);
         const float4 nw = make_float4(fmaf(keep[0], old.x, in[0]), fmaf(keep[1], old.y, in[1]), fmaf(keep[2], old.z, in[2]),
                                       fmaf(keep[3], old.w, in[3]));
         *sp = nw;
@@ -172,7 +209,7 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
           Tl<T>::st4((T*)p.qu + h * p.qu_z + tl_off<T>(m, o, p.d.dim64), v);
         } else if (nb < p.b_c) {
           const int dr = p.d.rot16 >> 4, b = nb - p.b_qr, h = b / dr, o = (b - h * dr) * 16 + 4 * kg;
-          const int slot = lm_slot(p.rows, m), pos = min(max(lm_pos(p.rows, m, slot), 0), p.rows.S - 1);
+          const int slot = PRE ? e_slot : lm_slot(p.rows, m), pos = min(max(PRE ? e_pos : lm_pos(p.rows, m, slot), 0), p.rows.S - 1);
           lm_rotate2(v, p.rope, pos, p.rot_pairs, o >> 1);
           Tl<T>::st4((T*)p.qr + h * p.qr_z + tl_off<T, 32>(m, o, p.d.rot32), v);
         } else if (nb < p.b_kr) {
@@ -180,7 +217,7 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
           *reinterpret_cast<float4*>(p.craw + (size_t)m * p.d.rank16 + o) = make_float4(v[0], v[1], v[2], v[3]);
         } else if (nb < p.b_g) {
           const int o = (nb - p.b_kr) * 16 + 4 * kg;
-          const int slot = lm_slot(p.rows, m), pos = lm_pos(p.rows, m, slot);
+          const int slot = PRE ? e_slot : lm_slot(p.rows, m), pos = PRE ? e_pos : lm_pos(p.rows, m, slot);
           if (pos >= 0 && pos < p.rows.S) {
             lm_rotate2(v, p.rope, pos, p.rot_pairs, o >> 1);
             Tl<T>::st4((T*)p.kr_cache + (size_t)slot * p.d.s64 * p.d.rot32 + tl_off<T, 32>(pos, o, p.d.rot32), v);
@@ -198,7 +235,7 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
       float sq = 0.f;
       if (live) {
         float4* xp = reinterpret_cast<float4*>(p.x + (size_t)m * p.d.w64 + n);
-        const float4 old = *xp;
+        const float4 old = PRE ? e_a : *xp;
         v[0] += old.x; v[1] += old.y; v[2] += old.z; v[3] += old.w;
         *xp = make_float4(v[0], v[1], v[2], v[3]);
         Tl<T>::st4((T*)p.xt + tl_off<T>(m, n, p.d.w64), v);
@@ -281,10 +318,10 @@ int launch_lm_gemm(int dtype, int epi, const LmGemm& g, int nz, hipStream_t st) 
 template <typename T>
 __global__ __launch_bounds__(256) void lm_embed_kernel(const int64_t* tokens, const T* table, float* x, T* xt, float* ssq,
                                                        int width, int w64, int np, int vocab) {
-  const int m = blockIdx.x;
+  const int m = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
   int64_t t = tokens[m];
   t = t < 0 ? 0 : (t >= vocab ? vocab - 1 : t);
-  for (int c = threadIdx.x; c < np * 16; c += 256) {  // np * 16 is a multiple of 16: a 16-lane group is whole or absent
+  if (c < np * 16) {  // a multiple of 16: a 16-lane group is whole or absent
     const float v = c < width ? El<T>::ld(table + (size_t)t * width + c) : 0.f;
     x[(size_t)m * w64 + c] = v;
     El<T>::st(xt + tl_off<T>(m, c, w64), v);
@@ -295,9 +332,9 @@ __global__ __launch_bounds__(256) void lm_embed_kernel(const int64_t* tokens, co
 int launch_lm_embed(int dtype, const int64_t* tokens, const void* table, float* x, void* xt, float* ssq, int rows, int width,
                     int w64, int np, int vocab, hipStream_t st) {
   if (dtype == VUI_DTYPE_F32)
-    hipLaunchKernelGGL(lm_embed_kernel<float>, dim3(rows), dim3(256), 0, st, tokens, (const float*)table, x, (float*)xt, ssq, width, w64, np, vocab);
+    hipLaunchKernelGGL(lm_embed_kernel<float>, dim3(rows, (np + 15) / 16), dim3(256), 0, st, tokens, (const float*)table, x, (float*)xt, ssq, width, w64, np, vocab);
   else
-    hipLaunchKernelGGL(lm_embed_kernel<bf16_t>, dim3(rows), dim3(256), 0, st, tokens, (const bf16_t*)table, x, (bf16_t*)xt, ssq, width, w64, np, vocab);
+    hipLaunchKernelGGL(lm_embed_kernel<bf16_t>, dim3(rows, (np + 15) / 16), dim3(256), 0, st, tokens, (const bf16_t*)table, x, (bf16_t*)xt, ssq, width, w64, np, vocab);
   HIP_TRY(hipGetLastError());
   return VUI_OK;
 }

@@ -15,14 +15,17 @@ __global__ __launch_bounds__(256) void scan_fold_kernel(const ScanArgs p, int nc
     p.agg[(size_t)nchunks * p.ld + ch] = make_float2(0.f, p.from_zero ? 0.f : p.state[ch]);
     return;
   }
-  const int t1 = min((c + 1) * LM_SCAN_CHUNK, p.T);
+  const int t0 = c * LM_SCAN_CHUNK;
+  float2 u[LM_SCAN_CHUNK];  // the whole chunk is requested at once
+#pragma unroll
+  for (int i = 0; i < LM_SCAN_CHUNK; ++i) u[i] = p.upd[(size_t)min(t0 + i, p.T - 1) * p.ld + ch];
   float a = 1.f, b = 0.f;
-#pragma unroll 8
-  for (int t = c * LM_SCAN_CHUNK; t < t1; ++t) {
-    const float2 u = p.upd[(size_t)t * p.ld + ch];
-    b = fmaf(u.x, b, u.y);
-    a *= u.x;
-  }
+#pragma unroll
+  for (int i = 0; i < LM_SCAN_CHUNK; ++i)
+    if (t0 + i < p.T) {
+      b = fmaf(u[i].x, b, u[i].y);
+      a *= u[i].x;
+    }
   p.agg[(size_t)c * p.ld + ch] = make_float2(a, b);
 }
 
@@ -30,23 +33,32 @@ template <typename T>
 __global__ __launch_bounds__(256) void scan_apply_kernel(const ScanArgs p, int nchunks) {
   const int ch = blockIdx.x * 256 + threadIdx.x, c = blockIdx.y;
   if (ch >= p.W) return;
+  const int t0 = c * LM_SCAN_CHUNK;
+  float2 u[LM_SCAN_CHUNK];
+  T g[LM_SCAN_CHUNK];
+#pragma unroll
+  for (int i = 0; i < LM_SCAN_CHUNK; ++i) {
+    const size_t o = (size_t)min(t0 + i, p.T - 1) * p.ld + ch;
+    u[i] = p.upd[o];
+    g[i] = ((const T*)p.gate)[o];
+  }
   float s;
   if (nchunks == 1) {
     s = p.from_zero ? 0.f : p.state[ch];
   } else {
     s = p.agg[(size_t)nchunks * p.ld + ch].y;
+#pragma unroll 8
     for (int k = 0; k < c; ++k) {
-      const float2 g = p.agg[(size_t)k * p.ld + ch];
-      s = fmaf(g.x, s, g.y);
+      const float2 f = p.agg[(size_t)k * p.ld + ch];
+      s = fmaf(f.x, s, f.y);
     }
   }
-  const int t1 = min((c + 1) * LM_SCAN_CHUNK, p.T);
-#pragma unroll 8
-  for (int t = c * LM_SCAN_CHUNK; t < t1; ++t) {
-    const float2 u = p.upd[(size_t)t * p.ld + ch];
-    s = fmaf(u.x, s, u.y);
-    El<T>::st((T*)p.act + tl_off<T>(t, ch, p.out_k), s * El<T>::ld((const T*)p.gate + (size_t)t * p.ld + ch));
-  }
+#pragma unroll
+  for (int i = 0; i < LM_SCAN_CHUNK; ++i)
+    if (t0 + i < p.T) {
+      s = fmaf(u[i].x, s, u[i].y);
+      El<T>::st((T*)p.act + tl_off<T>(t0 + i, ch, p.out_k), s * El<T>::ld(&g[i]));
+    }
   if (c == nchunks - 1) p.state[ch] = s;
 }
 

@@ -13,6 +13,8 @@
 
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 tl_bf16x8;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float tl_f32x4;
+// 16 bytes in flight: an array of HIP's uint4 structs that is filled and stored under conditions stays in scratch memory
+typedef __attribute__((__vector_size__(4 * sizeof(uint32_t)))) uint32_t tl_u32x4;
 
 template <typename T> struct Tl;
 template <> struct Tl<bf16_t> {
