@@ -105,7 +105,7 @@ int vui_lm_debug_layers(vui_lm_ctx* ctx, float* buf);
  * attending in the latent space (0 restores the default). */
 int vui_lm_expand_from(vui_lm_ctx* ctx, int rows);
 
-/* vui_sample_cb0 without a context: one token per row from fp32 logits (B, vocab), any vocabulary size. */
+/* vui_sample_cb0 without a context: one token per row from fp32 logits (B, vocab), vocab up to 524288. */
 int vui_sample_tokens(const float* logits, int vocab, float* rep_counts, int32_t* rep_hist, int32_t* rep_pos,
                       float penalty, int window, const vui_sample_params* sp, int64_t* out, int B, vui_stream_t stream);
 

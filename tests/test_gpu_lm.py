@@ -87,6 +87,27 @@ def test_prompt_against_token_by_token_and_portions(dt):
             assert e < tol, (cuts[:4], e)
 
 
+@BOTH
+def test_prompts_longer_than_one_native_call(dt, monkeypatch):
+    """Wanted places in any order, in several calls of at most 40 positions, some calls without any."""
+    from vui_amd.lm import TokenLM
+
+    monkeypatch.setattr(TokenLM, "PREFILL_CHUNK", 40)
+    cfg = U.mixed()
+    sd = U.weights(cfg, 28)
+    toks = U.tokens(131, cfg["vocab"], 15)
+    want = [130, 0, 79, 80, 39, 3]
+    eng = U.engine(cfg, sd, dt)
+    with eng.new_row() as row:
+        assert U.err(row.extend(toks, want), O.forward(cfg, sd, toks)[want]) < U.TOL[dt]
+        with pytest.raises(ValueError):
+            row.extend([1, 2], [2])
+        with pytest.raises(ValueError):
+            row.extend([], [])
+        with pytest.raises(ValueError):
+            row.extend(U.tokens(140, cfg["vocab"]))
+
+
 def test_both_forms_of_attention_agree():
     """Expanded keys against the latent space, from the same cache, for portions behind a long prefix (bf16)."""
     cfg = U.config([U.attn(), U.attn(heads=4, dim=40, vdim=24, kv_from=0)], ff=64)
@@ -376,3 +397,71 @@ def test_checkpoint_folder_and_trace_program(tmp_path):
         got = torch.from_numpy(np.fromfile(tmp_path / "out" / f"{step}.f32", dtype="<f4").reshape(len(want), -1).copy())
         assert U.err(got, ref[want]) < U.TOL[F32]
     assert not (tmp_path / "out" / "2.f32").exists()
+    p = subprocess.run([sys.executable, "-m", "vui_amd", "generate", "--model", str(tmp_path / "m"), "--dtype", "float32", "--tokens", "5,9,2",
+                        "--tokens", "7", "--max-new", "4"], capture_output=True, text=True, timeout=100, cwd=ROOT)
+    assert p.returncode == 0, p.stderr[-2000:]
+    got = [json.loads(ln) for ln in p.stdout.splitlines() if ln.startswith("{")]
+    assert got == [{"prompt": t, "tokens": O.greedy(cfg, sd, t, 4)} for t in ([5, 9, 2], [7])]
+
+
+def sample(logits, temperature, top_k, top_p, seed, frame, keep_ties=True, counts=None, penalty=1.0):
+    import ctypes as C
+
+    from vui_amd import _lib
+    from vui_amd.model import make_sample_params
+
+    lib = _lib.load(lm_only=True)
+    B, V = logits.shape
+    x = logits.float().cuda().contiguous()
+    ctr = torch.tensor([frame], dtype=torch.int32, device="cuda")
+    out = torch.full((B,), -1, dtype=torch.long, device="cuda")
+    sp = make_sample_params(temperature, top_k, seed, ctr, keep_ties=keep_ties, top_p=top_p or 0.0)
+    c = counts.cuda() if counts is not None else None
+    _lib.check(lib.vui_sample_tokens(x.data_ptr(), V, _lib.ptr(c), None, None, float(penalty), 0, C.byref(sp), out.data_ptr(), B,
+                                     torch.cuda.current_stream().cuda_stream), "vui_sample_tokens")
+    torch.cuda.synchronize()
+    return out.cpu().tolist(), c
+
+
+@pytest.mark.parametrize("V", [3000, 8193, 50257])
+def test_sampler_of_any_vocabulary(V):
+    """The register form up to 8192 entries and the re-reading form beyond, under the same rules: greedy (lowest index of
+    the maximum), top-k with ties kept and cut to exactly k, nucleus, both together, a penalty; heavy ties."""
+    from oracle import vui_oracle as VO
+
+    g = torch.Generator().manual_seed(V)
+    logits = torch.randn(12, V, generator=g) * 3
+    logits[4:8] = (logits[4:8] * 2).round() / 2  # many equal values
+    logits[0, [77, V - 1]] = 40.0
+    assert sample(logits, 1.0, 1, None, 0, 0)[0] == [int(r.argmax()) for r in logits]
+    agree = total = 0
+    for frame, (temp, k, p) in enumerate([(0.9, 50, None), (1.3, 0, None), (0.7, 0, 0.9), (1.0, 40, 0.8), (1.0, 5000 if V > 5000 else 900, 0.3), (1.0, 7, 0.999)]):
+        got, _ = sample(logits, temp, k, p, 99, frame)
+        for b, tok in enumerate(got):
+            u = VO.uniform01(99, frame, b, 0)
+            kept = VO.sample_codes_probs(logits[b], temp, k if k > 0 else None, p)
+            assert kept[tok] > 0, (V, temp, k, p, b)
+            agree += tok == VO._inverse_cdf(kept, u)
+            total += 1
+        if p is None and k > 0:
+            got, _ = sample(logits, temp, k, None, 7, frame, keep_ties=False)
+            for b, tok in enumerate(got):
+                kept = VO.cb0_probs(logits[b], temp, k)
+                assert kept[tok] > 0 and (kept > 0).sum() == k
+                agree += tok == VO._inverse_cdf(kept, VO.uniform01(7, frame, b, 0))
+                total += 1
+    assert agree >= 0.97 * total, (agree, total)
+    counts = torch.zeros(12, V)
+    counts[0, 77] = 3.0
+    got, after = sample(logits, 1.0, 1, None, 0, 0, counts=counts, penalty=2.0)
+    assert got[0] == V - 1 and after[0, V - 1] == 1.0 and after.sum() == 3.0 + 12
+
+
+def test_generation_with_a_large_vocabulary():
+    from vui_amd.lm_engine import TokenRequest
+
+    cfg = U.config([U.attn(), U.gru()], vocab=9001)
+    sd = U.weights(cfg, 27)
+    eng = U.engine(cfg, sd, max_rows=2, max_seq=40)
+    reqs = [TokenRequest(U.tokens(n, 9001, n), max_new=5) for n in (3, 20, 9)]
+    assert eng.generate(reqs) == [O.greedy(cfg, sd, r.tokens, 5) for r in reqs]

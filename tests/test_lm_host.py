@@ -212,6 +212,22 @@ def test_registry_chooses_by_config(tmp_path):
         registry.read_architecture(str(tmp_path / "missing"))
 
 
+# ---- command line ----
+def test_command_line_without_a_gpu(tmp_path, capsys):
+    from vui_amd.__main__ import main
+
+    assert main(["models"]) == 0
+    assert {ln.split("\t")[0] for ln in capsys.readouterr().out.splitlines()} == {"Sakupel", "Vui"}
+    (tmp_path / "config.json").write_text(json.dumps(U.mixed()))
+    assert main(["info", str(tmp_path)]) == 0
+    info = json.loads(capsys.readouterr().out)
+    assert info["architecture"] == "Sakupel" and info["layers"][2] == "latent_attention<-0" and info["layers"][1] == "mingru"
+    assert info["cached_values_per_token"] == 56 + 8 + 30 + 4 and info["state_bytes_per_row"] == 4 * (72 + 33)
+    assert main(["generate", "--model", str(tmp_path)]) == 2
+    with pytest.raises(SystemExit):
+        main(["trace", "--help"])
+
+
 # ---- trace replay ----
 def test_trace_replay_bookkeeping(tmp_path):
     from vui_amd.trace import replay

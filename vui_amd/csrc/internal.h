@@ -130,6 +130,7 @@ struct SampleArgs {
   int pad_from, pad_to;
 };
 int launch_sample(const SampleArgs& a, hipStream_t st);
+int launch_sample_wide(const SampleArgs& a, hipStream_t st);  // any vocabulary up to 524288 (sample_wide.hip)
 
 // x[b] = rnd(emb[code[b] + off] + pos_vec); optionally codes_out[b*stride] = code[b]
 int launch_rq_token(int dtype, const int64_t* code, int64_t off, const void* emb, const void* pos_vec, void* x,

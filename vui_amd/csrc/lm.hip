@@ -347,7 +347,7 @@ int vui_sample_tokens(const float* logits, int vocab, float* rep_counts, int32_t
   s.penalty = penalty; s.window = window; s.temperature = sp->temperature; s.top_k = sp->top_k; s.top_p = sp->top_p;
   s.seed = sp->seed; s.frame_ctr = sp->frame_ctr; s.state_rows = sp->state_rows; s.dev = sp->dev;
   s.exact_k = sp->keep_ties ? 0 : 1; s.CS = vocab; s.B = B; s.out = out; s.out_stride = 1;
-  return launch_sample(s, (hipStream_t)stream);
+  return vocab > 8192 ? launch_sample_wide(s, (hipStream_t)stream) : launch_sample(s, (hipStream_t)stream);  // what sample_kernel holds in registers
 }
 
 }  // extern "C"

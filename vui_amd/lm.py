@@ -97,6 +97,8 @@ class _NativeLM:
 
 @register_model("Sakupel")
 class TokenLM:
+    """Decoder-only token model: weights in the kernels' layout, prefill and decode over a slot cache."""
+
     PREFILL_CHUNK = 1024  # most positions of one native prefill call
 
     def __init__(self, config: LMConfig, state_dict: "dict[str, Tensor]", device="cuda", dtype=torch.bfloat16,
