@@ -73,11 +73,12 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const LatentArgs p) {
   Tl<T>::st4((T*)p.qlat + h * p.qlat_z + tl_off<T>(m, nb * 16 + 4 * (lane >> 4), p.d.rank64), v);
 }
 
-// A row that sees len keys is cut into pieces of this many (whole 32-key tiles, at least two), at most ns of them.
-__device__ __forceinline__ int latent_chunk(int len, int ns) { return max(((len + ns - 1) / ns + 31) & ~31, 64); }
+// A row that sees len keys is cut into pieces of this many (whole 32-key tiles), at most ns of them.  With more than
+// four rows a piece has two tiles at least: there are pieces enough, and fewer are merged faster.
+__device__ __forceinline__ int latent_chunk(int len, int ns, int M) { return max(((len + ns - 1) / ns + 31) & ~31, M > 4 ? 64 : 32); }
 // keys [lo, hi) of piece sp
-__device__ __forceinline__ void latent_range(int len, int ns, int sp, int& lo, int& hi) {
-  const int chunk = latent_chunk(len, ns);
+__device__ __forceinline__ void latent_range(int len, int ns, int M, int sp, int& lo, int& hi) {
+  const int chunk = latent_chunk(len, ns, M);
   lo = min(sp * chunk, len);
   hi = min(lo + chunk, len);
 }
@@ -96,7 +97,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(const LatentArgs p) {
   const int slot = lm_slot(p.rows, m);
   const int len = min(max(lm_pos(p.rows, m, slot) + 1, 1), p.rows.S);
   int lo, hi;
-  latent_range(len, p.n_splits, sp, lo, hi);
+  latent_range(len, p.n_splits, p.M, sp, lo, hi);
   if (lo >= hi) return;  // no such piece: latent_value_kernel does not look for it
   for (int k = tid; k < R + RR; k += 256)
     lq[k] = k < R ? (k < p.d.rank16 ? El<T>::ld((const T*)p.qlat + h * p.qlat_z + tl_off<T>(m, k, R)) : 0.f)
@@ -173,7 +174,7 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(const LatentArgs 
   const int slot = lm_slot(p.rows, m);
   const int len = min(max(lm_pos(p.rows, m, slot) + 1, 1), p.rows.S);
   int lo, hi;
-  latent_range(len, p.n_splits, sp, lo, hi);
+  latent_range(len, p.n_splits, p.M, sp, lo, hi);
   const tl_u32x4* cc = reinterpret_cast<const tl_u32x4*>((const bf16_t*)p.c_cache + (size_t)slot * p.d.s64 * (RK * 64));
   const tl_u32x4* kc = reinterpret_cast<const tl_u32x4*>((const bf16_t*)p.kr_cache + (size_t)slot * p.d.s64 * (RB * 32));
   if (lo >= hi) return;  // no such piece
@@ -292,7 +293,7 @@ __global__ __launch_bounds__(512) void latent_value_kernel(const LatentArgs p, i
     const int r = it / nk, k = (it - r * nk) * 64 + lane;
     const int m = m0 + r, slot = lm_slot(p.rows, m);
     const int len = min(max(lm_pos(p.rows, m, slot) + 1, 1), p.rows.S);
-    const int chunk = latent_chunk(len, ns), np = (len + chunk - 1) / chunk;  // pieces that exist
+    const int chunk = latent_chunk(len, ns, p.M), np = (len + chunk - 1) / chunk;  // pieces that exist
     const size_t piece = ((size_t)m * p.heads + h) * ns;
     const float2 ml = *reinterpret_cast<const float2*>(p.part_ml + 2 * (piece + min(lane, np - 1)));
     const float* pc = p.part + piece * R + k;
