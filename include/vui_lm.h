@@ -3,7 +3,7 @@
  * mixer, which sizes, which feed-forward) and run on the same library, slots and sampler as the Vui backbone.
  * No counterpart in the reference.
  *
- * A layer is parallel: x <- x + mixer(h) + ff(h) with h = norm(x), an RMS norm whose weight is one number.  The
+ * A layer is parallel: x <- x + mixer(h) + ff(h) with h = norm(x), an RMS norm with a scalar weight.  The
  * residual stream, norms, rotation angles, attention scores and weights, gates of a recurrence and its state are
  * fp32; products, cached latents and keys are of the context's dtype with fp32 accumulation.
  *
@@ -38,7 +38,7 @@ typedef struct vui_lm_config {
 typedef struct vui_lm_layer {
   int32_t mixer;      /* VUI_LM_* */
   /* latent attention: the cache holds per position the normed latent (kv_rank) and one rotated key part (rot_dim)
-   * shared by all heads; heads expand keys (dim) and values (vdim) from the latent */
+   * common to the heads; heads expand keys (dim) and values (vdim) from the latent */
   int32_t kv_from;    /* layer whose latents are read, or -1: the layer has a down-projection of its own */
   int32_t heads, dim, rot_dim, rot_pairs, vdim, kv_rank;
   float scale;
@@ -98,7 +98,7 @@ int vui_lm_decode(vui_lm_ctx* ctx, const int64_t* tokens, const int32_t* slot_id
 int vui_lm_prefill(vui_lm_ctx* ctx, const int64_t* tokens, int T, int slot, int pos0, int32_t* seq_lens,
                    const int32_t* want, int n_want, float* logits_out, vui_stream_t stream);
 
-/* Test aid: the residual stream after every layer of the calls that follow goes to buf (n_layers, rows of the call,
+/* Test aid: the residual stream behind each layer, for the calls that follow, goes to buf (n_layers, rows of the call,
  * width) fp32; NULL switches it off. */
 int vui_lm_debug_layers(vui_lm_ctx* ctx, float* buf);
 /* Test and measurement aid: positions of one call from which attention expands keys and values per head instead of

@@ -19,7 +19,7 @@ def rms_unit(x: Tensor, eps: float) -> Tensor:
 
 
 def scalar_norm(x: Tensor, g: Tensor, eps: float) -> Tensor:
-    """RMS norm whose weight is one number for all coordinates."""
+    """RMS norm with a scalar weight."""
     return rms_unit(x, eps) * g.reshape(())
 
 
@@ -39,7 +39,7 @@ def rotate_half(x: Tensor, pos: int, dims: int, base: float) -> Tensor:
 
 def latent_entries(h: Tensor, w: dict, p: str, mx: dict, eps: float) -> "tuple[Tensor, Tensor]":
     """What a layer with its own down-projection contributes per position: the normed latent (T, kv_rank) and the
-    rotated key part shared by all heads (T, rot_dim)."""
+    rotated key part common to the heads (T, rot_dim)."""
     y = h @ w[p + "dkv"].T
     c = rms_unit(y[:, :mx["kv_rank"]], eps) * w[p + "dkv.norm"]
     kr = torch.stack([rotate_half(y[t, mx["kv_rank"]:], t, mx["rot"]["dims"], mx["rot"]["base"]) for t in range(len(y))])
@@ -65,7 +65,7 @@ def latent_attention(h: Tensor, c: Tensor, kr: Tensor, w: dict, p: str, mx: dict
 
 
 def mingru(h: Tensor, w: dict, p: str, mx: dict) -> Tensor:
-    """Gated recurrence whose gate and candidate read only the current token."""
+    """S <- (1 - z) S + z cand, channel by channel; z and cand are functions of the token at hand alone."""
     z = torch.sigmoid(h @ w[p + "z"].T + w[p + "z.b"])
     u = h @ w[p + "x"].T + w[p + "x.b"]
     cand = torch.where(u >= 0, u + 0.5, torch.sigmoid(u))
@@ -87,7 +87,7 @@ def clamped_mlp(h: Tensor, w: dict, p: str, limit: float) -> Tensor:
 
 
 def forward(cfg: dict, w: dict, tokens, dtype=torch.float64, layers_out: "list | None" = None) -> Tensor:
-    """Logits (T, vocab) of one sequence.  layers_out, if given, receives the residual stream after every layer."""
+    """Logits (T, vocab) of one sequence.  layers_out, if given, receives the residual stream behind each layer."""
     w = {k: v.to(dtype) for k, v in w.items()}
     eps = cfg["norm"]["eps"]
     x = w["embed"][torch.as_tensor(tokens, dtype=torch.long)]

@@ -99,7 +99,7 @@ def main(argv=None) -> int:
     p.add_argument("path")
     p.set_defaults(run=cmd_info)
     p = sub.add_parser("generate")
-    p.add_argument("--model", required=True, help="folder with config.json and model.safetensors")
+    p.add_argument("--model", required=True, help="checkpoint folder (config.json, model.safetensors)")
     p.add_argument("--tokens", action="append", default=[], help="prompt as token ids, e.g. 1,2,3 (may be given several times)")
     p.add_argument("--tokens-file", help="one prompt of token ids a line")
     p.add_argument("--max-new", type=int, default=64)

@@ -140,7 +140,7 @@ class LatentAttentionConfig:
 
 @dataclass
 class MinGRUConfig:
-    """Gated recurrence of `width` channels whose gate and candidate read the current token only."""
+    """Recurrence S <- (1 - z) S + z c over `width` channels, z and c functions of the token at hand alone."""
 
     width: int
 

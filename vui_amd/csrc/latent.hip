@@ -1,5 +1,5 @@
 // Latent attention: per position the cache holds one normed latent c (kv_rank) and one rotated key part (rot_dim)
-// shared by all heads; head h's key is W_uk[h] c and its value W_uv[h] c.
+// common to the heads; head h's key is W_uk[h] c and its value W_uv[h] c.
 //
 // Two forms of the same sums.  Few rows attend in the latent space: the query goes through W_uk[h]^T once
 // (latent_query_kernel), scores are its products with the cached latents, the softmax average of the latents goes

@@ -140,7 +140,7 @@ class TokenLM:
 
     @classmethod
     def from_pretrained(cls, path: str, device="cuda", dtype=torch.bfloat16, **kw) -> "TokenLM":
-        """A local folder with config.json and model.safetensors."""
+        """A local checkpoint folder: config.json beside model.safetensors."""
         from safetensors.torch import load_file
 
         with open(os.path.join(path, "config.json")) as f:

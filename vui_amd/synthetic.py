@@ -113,18 +113,18 @@ def synthetic_codec_state_dict(cfg, seed: int = 0) -> dict[str, Tensor]:
 
 def token_lm_config(width: int, heads: int, ff: int, dim: int, rot_dim: int, vdim: int, kv_rank: int, n_layers: int,
                     vocab: int = 8192, rnn_width: int = 0) -> dict:
-    """A Sakupel configuration whose layers repeat the pattern: attention with latents of its own, attention on the same
-    latents, minGRU, attention with latents of its own."""
+    """A Sakupel configuration whose layers repeat the pattern: attention with own latents, minGRU, attention on the
+    latents of the first, attention with own latents."""
     layers = []
     own = 0
     for i in range(n_layers):
         mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
-        if i % 4 == 2:
+        if i % 4 == 1:
             layers.append({"type": "mingru", "mixer": {"width": rnn_width or width}, "mlp": mlp})
             continue
         mx = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank,
               "scale": (dim + rot_dim) ** -0.5, "rot": {"dims": rot_dim, "base": 10000.0}}
-        if i % 4 == 1:
+        if i % 4 == 2:
             mx["kv_from"] = own
         else:
             own = i

@@ -1,14 +1,14 @@
-"""Replays a trace: given token ids go through a model step by step, logits are written, nothing is sampled.
+"""Trace replay: known token ids are run as recorded steps and the logits of chosen places are kept.  No sampling.
 
-    bin/trace_run --model DIR --dtype bfloat16|float32 --out DIR --max-tokens N
+    bin/trace_run --model FOLDER --dtype float32 --out LOGITS --max-tokens 4096 < steps.jsonl
 
-Steps come from standard input, one JSON object a line:
+Every input line is one step in JSON:
 
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+    {"step": 12, "entries": [{"id": "r7", "tokens": [41, 8], "want": [1]}], "end": ["r7"]}
 
-`entries`: for each request its next tokens and the places among them whose logits are wanted; `end`: requests that
-are finished after the step.  A step in which something is wanted writes OUT/<step>.f32, the logits in the order of the
-entries and of `want` (little-endian fp32, [wanted, vocab]).  After every step `done <step>` is printed."""
+An entry continues (or starts) the request named by its id with these tokens; `want` picks places among them by index.  Requests
+named in `end` give their slot back once the step is through.  LOGITS/12.f32 then holds the picked rows one after the other as
+little-endian fp32 (no file for a step that picks none), and `done 12` on standard output says that it does."""
 from __future__ import annotations
 
 import argparse
@@ -56,10 +56,10 @@ def replay(engine, lines, out_dir: str, emit) -> None:
 
 def main(argv=None) -> int:
     ap = argparse.ArgumentParser(prog="trace_run", description="Replay a trace of token steps and write logits.")
-    ap.add_argument("--model", required=True, help="folder with config.json and model.safetensors")
+    ap.add_argument("--model", required=True, help="checkpoint folder (config.json, model.safetensors)")
     ap.add_argument("--dtype", default="bfloat16", choices=["bfloat16", "float32"])
     ap.add_argument("--out", required=True, help="folder for the logits")
-    ap.add_argument("--max-tokens", type=int, default=4096, help="most tokens live requests hold at any time")
+    ap.add_argument("--max-tokens", type=int, default=4096, help="positions to size a slot for")
     ap.add_argument("--max-rows", type=int, default=4, help="most requests alive at a time")
     args = ap.parse_args(argv)
     ensure_library()
