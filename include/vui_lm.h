@@ -3,9 +3,15 @@
  * mixer, which sizes, which feed-forward) and run on the same library, slots and sampler as the Vui backbone.
  * No counterpart in the reference.
  *
- * A layer is parallel: x <- x + mixer(h) + ff(h) with h = norm(x), an RMS norm with a scalar weight.  The
- * residual stream, norms, rotation angles, attention scores and weights, gates of a recurrence and its state are
- * fp32; products, cached latents and keys are of the context's dtype with fp32 accumulation.
+ * Two forms of layers (vui_lm_config.norm_groups):
+ *   parallel (0): x <- x + mixer(h) + ff(h) with h = norm(x), an RMS norm with a scalar weight;
+ *   sandwich (n >= 1): x <- x + norm(mixer(norm(x))), then x <- x + norm(ff(norm(x))), every norm over n equal
+ *     consecutive parts of the vector with one weight per entry.
+ * A model that runs some of its layers several times lists every run as a layer of its own: the same weights, but
+ * caches and states of its own.
+ *
+ * The residual stream, norms, positions and angles, attention scores and weights, routers, gates of a recurrence and
+ * its state are fp32; products, cached latents, keys and values are of the context's dtype with fp32 accumulation.
  *
  * Conventions as in vui_amd.h: caller-owned device memory, work enqueued on the given stream without waiting,
  * 0 or a negative VUI_E* code, vui_last_error().  vui_lm_decode may be recorded into a HIP graph.
@@ -22,9 +28,17 @@
 extern "C" {
 #endif
 
-#define VUI_LM_MAX_LAYERS 128
+#define VUI_LM_MAX_LAYERS 1024
+/* mixers; the first two belong to parallel layers, the others to sandwich layers */
 #define VUI_LM_LATENT_ATTENTION 0
 #define VUI_LM_MINGRU 1
+#define VUI_LM_GLA 2
+#define VUI_LM_SIGMOID_ATTENTION 3
+/* activations of an ungated feed-forward */
+#define VUI_LM_ACT_XIELU 0   /* z > 0: act_pos z^2 + z / 2, else act_neg (exp(z) - 1 - z) + z / 2 */
+#define VUI_LM_ACT_RELU2 1
+#define VUI_LM_MAX_TOP 16    /* experts a token uses */
+#define VUI_LM_MAX_EXPERTS 1024
 
 typedef struct vui_lm_config {
   int32_t dtype;      /* VUI_DTYPE_*: weights, activations and caches */
@@ -33,6 +47,8 @@ typedef struct vui_lm_config {
   int32_t n_slots;
   int32_t max_rows;   /* most positions of one vui_lm_prefill call (sizes the workspace) */
   float norm_eps;
+  int32_t norm_groups; /* 0: parallel layers; else sandwich layers with norms over this many parts */
+  float embed_scale;   /* sandwich layers: the embedding is multiplied by this */
 } vui_lm_config;
 
 typedef struct vui_lm_layer {
@@ -58,7 +74,31 @@ typedef struct vui_lm_layer {
   const float *bias_z, *bias_x; /* (gru16) */
   void* c_cache;          /* (n_slots, s64, rank64) tiled rows: latents; of layer kv_from when that is set */
   void* kr_cache;         /* (n_slots, s64, rot32) tiled rows (32-column blocks): rotated key parts */
-  float* state;           /* (n_slots, gru16) fp32 */
+  float* state;           /* (n_slots, gru16) fp32; gated linear attention (n_slots, heads, dim16, vdim16) */
+
+  /* ---- sandwich layers ----
+   * sigmoid attention (heads, kv_heads, dim, vdim, scale): queries and keys normed per head, the query times
+   * 1 + temp_coef ln(floor((p + 1) / temp_every) + 1) at position p, weights sigmoid(score scale + bias), where the
+   * bias is a table over the distance that stays at its last entry beyond it.
+   * gated linear attention (heads, dim, vdim, rank): S <- diag(a) S + k v^T, a = sigmoid(W_a2 W_a1 h + b)^inv_tau */
+  int32_t kv_heads, temp_every, bias_len, rank;
+  float temp_coef, inv_tau;
+  /* ungated feed-forward of ff features per expert; experts = 0: one dense feed-forward */
+  int32_t act, experts, top;
+  float act_pos, act_neg;
+  const float *norm1, *norm1b, *norm2, *norm2b; /* (w64), zero beyond width */
+  const float *in_bias, *out_bias;              /* (in_rows), (out_rows), or NULL */
+  const float *q_norm, *k_norm;                 /* (dim16) */
+  const float* dist_bias;                       /* (heads, bias_len): distances 0 .. bias_len - 1 and beyond */
+  void *k_cache;                                /* (n_slots, kv_heads, s64, dim64) tiled rows */
+  void *v_cache;                                /* (n_slots, kv_heads, s64 / 32, vdim16 / 16) blocks of 16 dims x 32 positions */
+  const float *w_a2, *a2_bias;                  /* (heads, dim16, rank), (heads, dim16) */
+  const float* head_norm;                       /* (vdim16) */
+  const void *w_up, *w_down;                    /* (experts or 1, ff16, w64), (experts or 1, out_rows, ff64) tiled */
+  const void* w_router;                         /* (experts16, w64) tiled */
+  const float* router_bias;                     /* (experts16) */
+  const void* loop_in;                          /* (out_rows, 2 w64) tiled or NULL: x <- loop_in [x; embedding] + loop_step ahead of the layer */
+  const float* loop_step;                       /* (w64) */
 } vui_lm_layer;
 
 /* Padded sizes of a layer's operands (all derived from the configuration). */
@@ -69,12 +109,13 @@ typedef struct vui_lm_dims {
   int32_t mix_rows, in_rows; /* rows of w_in: mixer part, all */
   int32_t ff_pad, ff_off;    /* feed-forward columns (padded) and where they start inside out_k */
   int32_t out_k, out_rows;
+  int32_t ff16, ff64, experts16;
 } vui_lm_dims;
 
 typedef struct vui_lm_weights {
   const void* embed;       /* (vocab, width) row-major */
   const void* head;        /* (vocab padded to 32, w64) tiled */
-  const float* final_norm; /* (1) */
+  const float* final_norm; /* (1); sandwich layers (w64) */
 } vui_lm_weights;
 
 typedef struct vui_lm_ctx vui_lm_ctx;
@@ -104,6 +145,9 @@ int vui_lm_debug_layers(vui_lm_ctx* ctx, float* buf);
 /* Test and measurement aid: positions of one call from which attention expands keys and values per head instead of
  * attending in the latent space (0 restores the default). */
 int vui_lm_expand_from(vui_lm_ctx* ctx, int rows);
+/* The same for sandwich layers: positions of one call from which attention takes blocks of a prompt, and a gated linear
+ * attention its chunked form (0 restores the defaults). */
+int vui_lm_block_from(vui_lm_ctx* ctx, int attn_rows, int gla_rows);
 
 /* vui_sample_cb0 without a context: one token per row from fp32 logits (B, vocab), vocab up to 524288. */
 int vui_sample_tokens(const float* logits, int vocab, float* rep_counts, int32_t* rep_hist, int32_t* rep_pos,

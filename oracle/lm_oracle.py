@@ -86,9 +86,129 @@ def clamped_mlp(h: Tensor, w: dict, p: str, limit: float) -> Tensor:
     return (g * torch.sigmoid(1.702 * g) * (u + 1)) @ w[p + "down"].T
 
 
+# ---- mechanisms of the design Mabidra ----
+def grouped_norm(x: Tensor, w: Tensor, groups: int, eps: float) -> Tensor:
+    """Every one of `groups` equal consecutive parts over its own root mean square, then one weight per entry."""
+    parts = x.reshape(*x.shape[:-1], groups, x.shape[-1] // groups)
+    return rms_unit(parts, eps).reshape(x.shape) * w
+
+
+def gated_linear_attention(h: Tensor, w: dict, p: str, mx: dict, eps: float) -> Tensor:
+    """S <- diag(a) S + k v^T per head, read by q; a decays the rows of S (one number per key channel); the read is
+    normed per head and multiplied by silu of a gate."""
+    T, H, dim, vdim = len(h), mx["heads"], mx["dim"], mx["vdim"]
+    q = (h @ w[p + "q"].T).reshape(T, H, dim) / math.sqrt(dim)
+    k = (h @ w[p + "k"].T).reshape(T, H, dim)
+    v = (h @ w[p + "v"].T).reshape(T, H, vdim)
+    z = h @ w[p + "a1"].T @ w[p + "a2"].T + w[p + "a2.b"]
+    a = torch.exp(torch.nn.functional.logsigmoid(z) / mx["tau"]).reshape(T, H, dim)
+    g = h @ w[p + "g"].T
+    S = torch.zeros(H, dim, vdim, dtype=h.dtype)
+    rows = []
+    for t in range(T):
+        S = a[t][:, :, None] * S + k[t][:, :, None] * v[t][:, None, :]
+        o = (S * q[t][:, :, None]).sum(dim=1)
+        rows.append((rms_unit(o, eps) * w[p + "norm"]).reshape(-1))
+    return (torch.stack(rows) * g * torch.sigmoid(g)) @ w[p + "o"].T
+
+
+def distance_bucket(n: int, buckets: int, far: int) -> int:
+    """Bucket of a distance n >= 0: one each below buckets / 2, then logarithmic, full at `far`."""
+    half = buckets // 2
+    if n < half:
+        return n
+    if far <= half:
+        return buckets - 1
+    return min(buckets - 1, half + math.floor(math.log(n / half) / math.log(far / half) * (buckets - half) + 1e-9))
+
+
+def sigmoid_attention(h: Tensor, w: dict, p: str, mx: dict, eps: float) -> Tensor:
+    """Causal attention whose weights are sigmoids of the scores: normed queries and keys, a temperature that grows with
+    the position, a bias per distance bucket and head, a number per head, a gate per head on the output."""
+    T, H, G, dim, vdim = len(h), mx["heads"], mx["kv_heads"], mx["dim"], mx["vdim"]
+    q = rms_unit((h @ w[p + "q"].T + w[p + "q.b"]).reshape(T, H, dim), eps) * w[p + "q.norm"]
+    k = rms_unit((h @ w[p + "k"].T + w[p + "k.b"]).reshape(T, G, dim), eps) * w[p + "k.norm"]
+    v = (h @ w[p + "v"].T + w[p + "v.b"]).reshape(T, G, vdim)
+    gate = torch.sigmoid(h @ w[p + "g"].T)
+    rel = w[p + "rel"]
+    bucket = torch.tensor([distance_bucket(n, len(rel), mx["bias_max"]) for n in range(T)])
+    qt = mx.get("q_temp")
+    out = torch.zeros(T, H, vdim, dtype=h.dtype)
+    for t in range(T):
+        temp = 1.0 + qt["coef"] * math.log((t + 1) // qt["every"] + 1) if qt else 1.0
+        for a in range(H):
+            b = a // (H // G)
+            s = (k[:t + 1, b] @ (q[t, a] * temp)) * mx["scale"] + rel[bucket[:t + 1].flip(0), a] + w[p + "pb"][a]
+            out[t, a] = torch.sigmoid(s) @ v[:t + 1, b] * gate[t, a]
+    return out.reshape(T, H * vdim) @ w[p + "o"].T + w[p + "o.b"]
+
+
+def xielu(z: Tensor, p: Tensor, q: Tensor) -> Tensor:
+    """Quadratic above zero, exponential below, slope 1/2 at zero; p and q pass through softplus."""
+    sp = torch.nn.functional.softplus
+    neg = torch.clamp(z, max=0.0)
+    return torch.where(z > 0, sp(p) * z * z, (0.5 + sp(q)) * (torch.expm1(neg) - neg)) + z / 2
+
+
+def xielu_mlp(h: Tensor, w: dict, p: str) -> Tensor:
+    return xielu(h @ w[p + "up"].T, *w[p + "act"]) @ w[p + "down"].T
+
+
+def expert_mlp(h: Tensor, w: dict, p: str, router: dict) -> Tensor:
+    """The `top` experts with the largest router logits per token, weighed by a softmax over those; relu squared inside."""
+    z = h @ w[p + "router"].T + w[p + "router.b"]
+    out = torch.zeros_like(h)
+    for t in range(len(h)):
+        best = torch.topk(z[t], router["top"])
+        share = torch.softmax(best.values, 0)
+        for e, s in zip(best.indices.tolist(), share):
+            out[t] += s * (torch.relu(h[t] @ w[f"{p}e{e}.up"].T).square() @ w[f"{p}e{e}.down"].T)
+    return out
+
+
+def layer_passes(cfg: dict) -> "list[tuple[int, int | None]]":
+    """The layers in the order they run: (layer, number of the pass it starts, or None)."""
+    n, loop = len(cfg["layers"]), cfg.get("loop")
+    if not loop:
+        return [(i, None) for i in range(n)]
+    order = [(i, None) for i in range(loop["start"])]
+    for t in range(loop["times"]):
+        order += [(i, t if i == loop["start"] else None) for i in range(loop["start"], loop["stop"])]
+    return order + [(i, None) for i in range(loop["stop"], n)]
+
+
+def forward_sandwich(cfg: dict, w: dict, tokens, layers_out: "list | None" = None) -> Tensor:
+    """Mabidra: norms on both sides of every sublayer, a loop over some layers that mixes the embedding back in."""
+    eps, groups = cfg["norm"]["eps"], cfg["norm"]["groups"]
+    x = x0 = w["embed"][torch.as_tensor(tokens, dtype=torch.long)] * cfg["embedding"]["scale"]
+    for i, start in layer_passes(cfg):
+        p, layer = f"l{i}.", cfg["layers"][i]
+        mx = layer["mixer"]
+        if start is not None:
+            x = torch.cat((x, x0), dim=-1) @ w["loop.in"].T + w["loop.step"][start]
+        h = grouped_norm(x, w[p + "norm1"], groups, eps)
+        if layer["type"] == "gla":
+            y = gated_linear_attention(h, w, p + "mix.", mx, eps)
+        elif layer["type"] == "attention":
+            y = sigmoid_attention(h, w, p + "mix.", mx, eps)
+        else:
+            raise ValueError(layer["type"])
+        x = x + grouped_norm(y, w[p + "norm1b"], groups, eps)
+        mlp = layer.get("mlp")
+        if mlp is not None:
+            h = grouped_norm(x, w[p + "norm2"], groups, eps)
+            y = xielu_mlp(h, w, p + "mlp.") if mlp["kind"] == "dense" else expert_mlp(h, w, p + "mlp.", mlp["router"])
+            x = x + grouped_norm(y, w[p + "norm2b"], groups, eps)
+        if layers_out is not None:
+            layers_out.append(x.clone())
+    return grouped_norm(x, w["final.norm"], groups, eps) @ w["head"].T
+
+
 def forward(cfg: dict, w: dict, tokens, dtype=torch.float64, layers_out: "list | None" = None) -> Tensor:
     """Logits (T, vocab) of one sequence.  layers_out, if given, receives the residual stream behind each layer."""
     w = {k: v.to(dtype) for k, v in w.items()}
+    if cfg["architecture"] == "Mabidra":
+        return forward_sandwich(cfg, w, tokens, layers_out)
     eps = cfg["norm"]["eps"]
     x = w["embed"][torch.as_tensor(tokens, dtype=torch.long)]
     entries: dict = {}

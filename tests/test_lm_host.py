@@ -217,7 +217,7 @@ def test_command_line_without_a_gpu(tmp_path, capsys):
     from vui_amd.__main__ import main
 
     assert main(["models"]) == 0
-    assert {ln.split("\t")[0] for ln in capsys.readouterr().out.splitlines()} == {"Sakupel", "Vui"}
+    assert {ln.split("\t")[0] for ln in capsys.readouterr().out.splitlines()} == {"Mabidra", "Sakupel", "Vui"}
     (tmp_path / "config.json").write_text(json.dumps(U.mixed()))
     assert main(["info", str(tmp_path)]) == 0
     info = json.loads(capsys.readouterr().out)

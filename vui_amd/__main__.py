@@ -28,7 +28,7 @@ def cmd_models(args) -> int:
 
 
 def cmd_info(args) -> int:
-    from .config import Config, LatentAttentionConfig, LMConfig
+    from .config import Config, GatedLinearAttentionConfig, LatentAttentionConfig, LMConfig, SigmoidAttentionConfig
     from .registry import DEFAULT, read_architecture
 
     arch = read_architecture(args.path)
@@ -45,11 +45,17 @@ def cmd_info(args) -> int:
             c = LMConfig.from_dict(json.load(f))
         per_token = per_row = 0
         kinds = []
-        for layer in c.layers:
-            mx = layer.mixer
+        for i, _ in c.runs():
+            mx = c.layers[i].mixer
             if isinstance(mx, LatentAttentionConfig):
                 kinds.append("latent_attention" if mx.kv_from is None else f"latent_attention<-{mx.kv_from}")
                 per_token += mx.kv_rank + mx.rot_dim if mx.kv_from is None else 0
+            elif isinstance(mx, SigmoidAttentionConfig):
+                kinds.append("sigmoid_attention")
+                per_token += mx.kv_heads * (mx.dim + mx.vdim)
+            elif isinstance(mx, GatedLinearAttentionConfig):
+                kinds.append("gla")
+                per_row += 4 * mx.heads * mx.dim * mx.vdim
             else:
                 kinds.append("mingru")
                 per_row += 4 * mx.width

@@ -69,21 +69,26 @@ class CodecConfigC(C.Structure):
 class LmConfigC(C.Structure):
     """vui_lm_config (include/vui_lm.h)."""
     _fields_ = [(n, C.c_int32) for n in ("dtype", "width", "vocab", "n_layers", "max_seqlen", "n_slots", "max_rows")] + [
-        ("norm_eps", C.c_float)]
+        ("norm_eps", C.c_float), ("norm_groups", C.c_int32), ("embed_scale", C.c_float)]
 
 
 class LmLayerC(C.Structure):
     """vui_lm_layer."""
     _fields_ = [(n, C.c_int32) for n in ("mixer", "kv_from", "heads", "dim", "rot_dim", "rot_pairs", "vdim", "kv_rank")] + [
         ("scale", C.c_float), ("rnn_width", C.c_int32), ("ff", C.c_int32), ("limit", C.c_float)] + [(n, C.c_void_p) for n in (
-            "norm", "w_in", "w_out", "w_uk_t", "w_uk", "w_uv", "latent_norm", "rope", "bias_z", "bias_x", "c_cache", "kr_cache", "state")]
+            "norm", "w_in", "w_out", "w_uk_t", "w_uk", "w_uv", "latent_norm", "rope", "bias_z", "bias_x", "c_cache", "kr_cache", "state")] + [
+                (n, C.c_int32) for n in ("kv_heads", "temp_every", "bias_len", "rank")] + [("temp_coef", C.c_float), ("inv_tau", C.c_float)] + [
+                (n, C.c_int32) for n in ("act", "experts", "top")] + [("act_pos", C.c_float), ("act_neg", C.c_float)] + [
+                (n, C.c_void_p) for n in (
+                    "norm1", "norm1b", "norm2", "norm2b", "in_bias", "out_bias", "q_norm", "k_norm", "dist_bias", "k_cache", "v_cache",
+                    "w_a2", "a2_bias", "head_norm", "w_up", "w_down", "w_router", "router_bias", "loop_in", "loop_step")]
 
 
 class LmDimsC(C.Structure):
     """vui_lm_dims."""
     _fields_ = [(n, C.c_int32) for n in (
         "w16", "w64", "s64", "dim16", "dim64", "rot16", "rot32", "rank16", "rank64", "vdim16", "heads16", "gru16",
-        "mix_rows", "in_rows", "ff_pad", "ff_off", "out_k", "out_rows")]
+        "mix_rows", "in_rows", "ff_pad", "ff_off", "out_k", "out_rows", "ff16", "ff64", "experts16")]
 
 
 class LmWeightsC(C.Structure):
@@ -91,7 +96,8 @@ class LmWeightsC(C.Structure):
     _fields_ = [("embed", C.c_void_p), ("head", C.c_void_p), ("final_norm", C.c_void_p)]
 
 
-LM_LATENT_ATTENTION, LM_MINGRU = 0, 1
+LM_LATENT_ATTENTION, LM_MINGRU, LM_GLA, LM_SIGMOID_ATTENTION = range(4)
+LM_ACT_XIELU, LM_ACT_RELU2 = 0, 1
 
 
 # name -> (restype, argtypes); every symbol include/*.h declares
@@ -146,6 +152,7 @@ SIGNATURES = {
     "vui_lm_prefill": (_I, [_P, _P, _I, _I, _I, _P, _P, _I, _P, _P]),
     "vui_lm_debug_layers": (_I, [_P, _P]),
     "vui_lm_expand_from": (_I, [_P, _I]),
+    "vui_lm_block_from": (_I, [_P, _I, _I]),
     "vui_sample_tokens": (_I, [_P, _I, _P, _P, _P, _F, _I, C.POINTER(SampleParamsC), _P, _I, _P]),
     "vui_sample_logits": (_I, [_P, _P, _I, C.POINTER(SampleParamsC), _I, _P, _I, _P]),
 }

@@ -11,9 +11,11 @@ CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libvui_amd.so")
 # the token language models alone: their kernels, the sampler, the graph helpers
 LM_LIB = os.path.join(HERE, "libvui_lm.so")
-LM_SOURCES = ["runtime.hip", "misc.hip", "sample_wide.hip", "lm_gemm.hip", "latent.hip", "scan.hip", "lm.hip"]
+LM_SOURCES = ["runtime.hip", "misc.hip", "sample_wide.hip", "lm_gemm.hip", "latent.hip", "scan.hip", "rows.hip", "sigattn.hip",
+              "gla.hip", "moe.hip", "sandwich.hip", "lm.hip"]
 SOURCES = ["gemv.hip", "gemm16.hip", "attn.hip", "misc.hip", "frame.hip", "rqbatch.hip", "bbatch.hip", "prefill.hip", "codec.hip", "api.hip",
-           "runtime.hip", "sample_wide.hip", "lm_gemm.hip", "latent.hip", "scan.hip", "lm.hip"]
+           "runtime.hip", "sample_wide.hip", "lm_gemm.hip", "latent.hip", "scan.hip", "rows.hip", "sigattn.hip", "gla.hip", "moe.hip",
+           "sandwich.hip", "lm.hip"]
 FLAGS = [
     "-O3", "--offload-arch=gfx950", "-fPIC", "-std=c++17", "-Wall", "-Wno-unused-function",
     # packed-fp32 instructions are kept out of every code object of this library

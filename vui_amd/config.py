@@ -146,6 +146,38 @@ class MinGRUConfig:
 
 
 @dataclass
+class QueryTempConfig:
+    """The query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1)."""
+
+    coef: float
+    every: int
+
+
+@dataclass
+class SigmoidAttentionConfig:
+    """Causal attention whose weights are sigmoids of the scores.  heads query heads share kv_heads keys and values;
+    queries and keys are normed; the bias over the distance is a table by buckets, full at bias_max."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    bias_max: int
+    q_temp: QueryTempConfig | None = None
+
+
+@dataclass
+class GatedLinearAttentionConfig:
+    """Recurrence S <- diag(a) S + k v^T per head with a decay per key channel, a = sigmoid(z)^(1 / tau)."""
+
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+
+
+@dataclass
 class GatedMLPConfig:
     """Gated feed-forward with clamped branches."""
 
@@ -154,45 +186,148 @@ class GatedMLPConfig:
 
 
 @dataclass
+class XieluMLPConfig:
+    """Ungated feed-forward with xIELU, whose two constants are weights."""
+
+    ff: int
+
+
+@dataclass
+class ExpertsMLPConfig:
+    """`top` of `experts` ungated feed-forwards of ff features (relu squared) per token."""
+
+    ff: int
+    experts: int
+    top: int
+
+
+@dataclass
+class LoopConfig:
+    """Layers start .. stop - 1 run `times` times in a row."""
+
+    start: int
+    stop: int
+    times: int
+
+
+@dataclass
 class LMLayerConfig:
-    mixer: "LatentAttentionConfig | MinGRUConfig"
-    mlp: GatedMLPConfig | None = None
+    mixer: "LatentAttentionConfig | MinGRUConfig | SigmoidAttentionConfig | GatedLinearAttentionConfig"
+    mlp: "GatedMLPConfig | XieluMLPConfig | ExpertsMLPConfig | None" = None
+
+
+@dataclass(frozen=True)
+class LMDesign:
+    """What a design fixes: the form of its layers, the mixers (by the names its configuration uses) and the
+    feed-forwards it is made of."""
+
+    sandwich: bool
+    mixers: "dict[str, type]"
+    mlps: "dict[str, type]"
+
+
+LM_DESIGNS = {
+    "Sakupel": LMDesign(False, {"latent_attention": LatentAttentionConfig, "mingru": MinGRUConfig}, {"dense": GatedMLPConfig}),
+    "Mabidra": LMDesign(True, {"attention": SigmoidAttentionConfig, "gla": GatedLinearAttentionConfig},
+                        {"dense": XieluMLPConfig, "moe": ExpertsMLPConfig}),
+}
+
+
+def _latent_attention(i: int, mx: dict, layers: "list[LMLayerConfig]") -> LatentAttentionConfig:
+    mixer = LatentAttentionConfig(**{k: mx[k] for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "scale")},
+                                  rot=_from_dict(RotaryConfig, mx["rot"]), kv_from=mx.get("kv_from"))
+    if mixer.rot.dims > mixer.rot_dim or mixer.rot.dims % 2:
+        raise ValueError(f"layer {i}: cannot rotate {mixer.rot.dims} of {mixer.rot_dim} dims")
+    if mixer.kv_from is not None:
+        src = layers[mixer.kv_from].mixer if 0 <= mixer.kv_from < i else None
+        if not isinstance(src, LatentAttentionConfig) or src.kv_from is not None:
+            raise ValueError(f"layer {i}: kv_from={mixer.kv_from} names no earlier layer with latents of its own")
+        if (src.kv_rank, src.rot_dim, src.rot) != (mixer.kv_rank, mixer.rot_dim, mixer.rot):
+            raise ValueError(f"layer {i}: latents of layer {mixer.kv_from} have another shape or rotation")
+    return mixer
+
+
+def _sigmoid_attention(i: int, mx: dict) -> SigmoidAttentionConfig:
+    qt = mx.get("q_temp")
+    mixer = SigmoidAttentionConfig(**{k: mx[k] for k in ("heads", "kv_heads", "dim", "vdim", "scale", "bias_max")},
+                                   q_temp=None if qt is None else QueryTempConfig(coef=qt["coef"], every=qt["every"]))
+    if mixer.kv_heads < 1 or mixer.heads % mixer.kv_heads:
+        raise ValueError(f"layer {i}: {mixer.heads} heads cannot share {mixer.kv_heads} keys and values")
+    if mixer.q_temp is not None and mixer.q_temp.every < 1:
+        raise ValueError(f"layer {i}: q_temp.every={mixer.q_temp.every}")
+    return mixer
 
 
 @dataclass
 class LMConfig:
-    """A decoder-only token model: config.json's `layers` (type, mixer, mlp), `norm.eps`, `vocab`, `width`."""
+    """A decoder-only token model: config.json's `layers` (type, mixer, mlp), `norm`, `vocab`, `width`; for sandwich
+    layers also `embedding.scale`, `norm.groups` and `loop`."""
 
     architecture: str
     width: int
     vocab: int
     norm_eps: float
     layers: "list[LMLayerConfig]"
+    norm_groups: int = 0
+    embed_scale: float = 1.0
+    loop: LoopConfig | None = None
+
+    @property
+    def design(self) -> LMDesign:
+        return LM_DESIGNS[self.architecture]
+
+    def runs(self) -> "list[tuple[int, int | None]]":
+        """Every layer run in order: (layer, pass of the loop that starts with it, or None)."""
+        n = len(self.layers)
+        if self.loop is None:
+            return [(i, None) for i in range(n)]
+        a, b = self.loop.start, self.loop.stop
+        body = [(i, t if i == a else None) for t in range(self.loop.times) for i in range(a, b)]
+        return [(i, None) for i in range(a)] + body + [(i, None) for i in range(b, n)]
 
     @classmethod
     def from_dict(cls, d: dict) -> "LMConfig":
+        arch = d["architecture"]
+        if arch not in LM_DESIGNS:
+            raise ValueError(f"{arch!r} is not a design of token models")
+        design = LM_DESIGNS[arch]
         layers: "list[LMLayerConfig]" = []
         for i, e in enumerate(d["layers"]):
             mx = e["mixer"]
-            if e["type"] == "latent_attention":
-                mixer = LatentAttentionConfig(**{k: mx[k] for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "scale")},
-                                              rot=_from_dict(RotaryConfig, mx["rot"]), kv_from=mx.get("kv_from"))
-                if mixer.rot.dims > mixer.rot_dim or mixer.rot.dims % 2:
-                    raise ValueError(f"layer {i}: cannot rotate {mixer.rot.dims} of {mixer.rot_dim} dims")
-                if mixer.kv_from is not None:
-                    src = layers[mixer.kv_from].mixer if 0 <= mixer.kv_from < i else None
-                    if not isinstance(src, LatentAttentionConfig) or src.kv_from is not None:
-                        raise ValueError(f"layer {i}: kv_from={mixer.kv_from} names no earlier layer with latents of its own")
-                    if (src.kv_rank, src.rot_dim, src.rot) != (mixer.kv_rank, mixer.rot_dim, mixer.rot):
-                        raise ValueError(f"layer {i}: latents of layer {mixer.kv_from} have another shape or rotation")
-            elif e["type"] == "mingru":
+            kind = design.mixers.get(e["type"])
+            if kind is LatentAttentionConfig:
+                mixer = _latent_attention(i, mx, layers)
+            elif kind is MinGRUConfig:
                 mixer = MinGRUConfig(width=mx["width"])
+            elif kind is SigmoidAttentionConfig:
+                mixer = _sigmoid_attention(i, mx)
+            elif kind is GatedLinearAttentionConfig:
+                mixer = GatedLinearAttentionConfig(**{k: mx[k] for k in ("heads", "dim", "vdim", "tau")})
             else:
                 raise ValueError(f"layer {i}: unknown mixer {e['type']!r}")
             mlp = None
             if e.get("mlp") is not None:
-                if e["mlp"].get("kind", "dense") != "dense":
-                    raise ValueError(f"layer {i}: unknown feed-forward {e['mlp']['kind']!r}")
-                mlp = GatedMLPConfig(ff=e["mlp"]["ff"], limit=e["mlp"]["limit"])
+                ff = e["mlp"]
+                kind = design.mlps.get(ff.get("kind", "dense"))
+                if kind is GatedMLPConfig:
+                    mlp = GatedMLPConfig(ff=ff["ff"], limit=ff["limit"])
+                elif kind is XieluMLPConfig:
+                    mlp = XieluMLPConfig(ff=ff["ff"])
+                elif kind is ExpertsMLPConfig:
+                    mlp = ExpertsMLPConfig(ff=ff["expert"]["ff"], experts=ff["router"]["experts"], top=ff["router"]["top"])
+                    if not 1 <= mlp.top <= mlp.experts:
+                        raise ValueError(f"layer {i}: cannot use {mlp.top} of {mlp.experts} experts")
+                else:
+                    raise ValueError(f"layer {i}: unknown feed-forward {ff['kind']!r}")
             layers.append(LMLayerConfig(mixer, mlp))
-        return cls(architecture=d["architecture"], width=d["width"], vocab=d["vocab"], norm_eps=d["norm"]["eps"], layers=layers)
+        out = cls(architecture=arch, width=d["width"], vocab=d["vocab"], norm_eps=d["norm"]["eps"], layers=layers)
+        if design.sandwich:
+            out.norm_groups = d["norm"].get("groups", 1)
+            out.embed_scale = (d.get("embedding") or {}).get("scale", 1.0)
+            if out.norm_groups < 1 or out.width % out.norm_groups:
+                raise ValueError(f"a width of {out.width} has no {out.norm_groups} equal parts")
+            if d.get("loop") is not None:
+                out.loop = _from_dict(LoopConfig, d["loop"])
+                if not (0 <= out.loop.start < out.loop.stop <= len(layers) and out.loop.times >= 1):
+                    raise ValueError(f"loop over layers {out.loop.start} .. {out.loop.stop - 1} of {len(layers)}")
+        return out

@@ -1,6 +1,9 @@
-// Internal interface between the kernels of the token language models (lm_gemm.hip, latent.hip, scan.hip) and their
-// step (lm.hip).
+// Internal interface between the kernels of the token language models and their step: lm.hip (context, parallel layers),
+// sandwich.hip (sandwich layers), lm_gemm.hip (products), latent.hip and sigattn.hip (attention), scan.hip and gla.hip
+// (recurrences), rows.hip (residual rows and norms), moe.hip (expert routing).
 #pragma once
+#include <vector>
+
 #include "../../include/vui_lm.h"
 #include "internal.h"
 
@@ -29,6 +32,13 @@ enum {
   LM_LOGITS,        // fp32 logits of chosen rows
   LM_EXPAND_K,      // keys of one head per blockIdx.z from cached latents
   LM_EXPAND_V,      // values, transposed
+  // sandwich layers (rows arrive normed)
+  LM_HEAD,          // LM_LOGITS without a row scale
+  LM_PROJ,          // W x + bias in the context's dtype, row-major
+  LM_PLAIN,         // the same in fp32
+  LM_ACT,           // activation of an ungated feed-forward, tiled
+  LM_MOE_UP,        // LM_ACT of the rows an expert was given, by tiles of the expert-sorted entries
+  LM_MOE_DOWN,      // LM_PLAIN from those, one output row per (row, choice)
 };
 
 struct LmGemm {
@@ -75,6 +85,15 @@ struct LmGemm {
   // expansion
   void* kv_out;
   size_t kv_z;
+  // sandwich layers
+  void* out;       // (rows, ldo) of the epilogue's type
+  int ldo;
+  const float* bias;  // (N) or nullptr
+  int act_kind, act_k;  // VUI_LM_ACT_*, columns of act
+  float act_pos, act_neg;
+  // entries (row top + choice) sorted by expert, every expert's padded with -1 to whole tiles; expert of each tile
+  const int32_t *ent, *tile_e, *n_tiles;
+  int top, max_tiles;
 };
 int launch_lm_gemm(int dtype, int epi, const LmGemm& g, int nz, hipStream_t st);
 int launch_lm_embed(int dtype, const int64_t* tokens, const void* table, float* x, void* xt, float* ssq, int rows, int width,
@@ -128,3 +147,114 @@ struct ScanArgs {
 };
 int launch_gated_scan(const ScanArgs& a, hipStream_t st);
 #define LM_SCAN_CHUNK 32
+
+// ---- residual rows of sandwich layers (rows.hip) ----
+struct RowArgs {
+  int dtype, M, width, w64, ldy, groups;
+  float eps;
+  // what the residual becomes, in this order of precedence
+  const int64_t* tokens;   // embedding rows times emb_scale, copied to the second half of xcat too
+  const void* embed;
+  int vocab;
+  float emb_scale;
+  const float* step;       // y + step
+  const float* post;       // x + norm(y) post; y the sum over `top` rows weighed by share, or one row (share nullptr)
+  const float* y;
+  const float* share;      // (M, top)
+  int top;
+  float* x;                // (rows, w64)
+  float* layer_out;        // (M, width) or nullptr
+  // what is left for the next product: the normed row, or the row itself in the first half of xcat
+  const float* next;       // (w64) weight, or nullptr
+  void* xt;                // (rows, w64) tiled
+  void* xcat;              // (rows, 2 w64) tiled: [x | embedding]
+  int to_cat;
+};
+int launch_lm_rows(const RowArgs& a, hipStream_t st);
+
+// ---- attention with sigmoid weights (sigattn.hip) ----
+struct SigAttnArgs {
+  int dtype, M, heads, kv_heads, dim, vdim;
+  float scale, eps;
+  LmRows rows;
+  vui_lm_dims d;
+  const void* raw;         // (rows, ld): per head query, per group key and value, per head gate
+  int ld;
+  const float *q_norm, *k_norm;
+  float temp_coef;
+  int temp_every;
+  const float* bias;       // (heads, bias_len)
+  int bias_len;
+  void *k_cache, *v_cache;
+  void* q;                 // (heads, rows, dim64) tiled
+  size_t q_z;
+  float* part;             // (rows, heads, n_splits, vdim16)
+  int n_splits;
+  void* act;               // (rows, out_k) tiled
+};
+int launch_sig_prep(const SigAttnArgs& a, hipStream_t st);    // norms, temperature, append
+int launch_sig_pieces(const SigAttnArgs& a, hipStream_t st);  // few rows: pieces, merge, gate
+int launch_sig_prompt(const SigAttnArgs& a, hipStream_t st);  // block of one sequence, bf16
+bool sig_mfma_ok(const vui_lm_dims& d);
+int sig_splits(int M, int heads, int kv_heads);
+
+// ---- gated linear attention (gla.hip) ----
+struct GlaArgs {
+  int dtype, M, heads, dim, vdim, rank;
+  float eps, inv_tau, q_scale;
+  LmRows rows;
+  vui_lm_dims d;
+  const void* raw;         // (rows, ld): per head query, key, value, gate; the low-rank part of the decay
+  int ld;
+  const float *w_a2, *a2_bias, *head_norm;
+  float* state;            // (n_slots, heads, dim16, vdim16)
+  float *bsum, *upd, *dec; // chunked form: (rows, heads, dim16), (chunks, heads, dim16, vdim16), (chunks, heads, dim16)
+  void* act;
+};
+int launch_gla_step(const GlaArgs& a, hipStream_t st);   // one position per slot, or the positions of one sequence in turn
+int launch_gla_chunk(const GlaArgs& a, hipStream_t st);  // positions of one sequence by chunks
+bool gla_chunk_ok(const vui_lm_dims& d);
+#define LM_GLA_CHUNK 32
+
+// ---- expert routing (moe.hip) ----
+struct RouteArgs {
+  int M, E, ldl, top, tile_rows;
+  const float* logits;     // (M, ldl)
+  int32_t* choice;         // (M, top)
+  float* share;            // (M, top)
+  int32_t *ent, *tile_e, *n_tiles;
+};
+int launch_moe_route(const RouteArgs& a, hipStream_t st);
+static inline int moe_max_tiles(int entries, int experts, int tile_rows) {
+  const int a = entries / tile_rows + experts;
+  return entries < a ? entries : a;
+}
+
+// ---- context ----
+struct vui_lm_ctx {
+  vui_lm_config c;
+  vui_lm_weights w;
+  std::vector<vui_lm_layer> layers;
+  std::vector<vui_lm_dims> dims;
+  int R16;  // rows of the activation buffers
+  float* x; void* xt; float* ssq;
+  void *qu, *qr, *qlat;
+  float *craw, *gate, *part, *part_ml;
+  void* act;
+  float2* upd; void* sg; float2* agg;
+  void *kx, *vx;
+  float* layers_out;
+  int expand_from;
+  // sandwich layers
+  void *xcat, *raw, *ffa;
+  float *y, *bsum, *gupd, *gdec, *rlog, *share;
+  int32_t *choice, *ent, *tile_e, *n_tiles;
+  int attn_from, gla_from;
+};
+static inline int lm_pad(int v, int a) { return (v + a - 1) / a * a; }
+static inline size_t lm_esz(const vui_lm_config& c) { return c.dtype == VUI_DTYPE_F32 ? 4 : 2; }
+int sandwich_layer_dims(const vui_lm_config& c, const vui_lm_layer& L, vui_lm_dims* o);
+int sandwich_check_layer(const vui_lm_config& c, const vui_lm_layer& L, int l);
+bool sandwich_pointers_ok(const vui_lm_config& c, const vui_lm_layer& L);
+size_t sandwich_carve(const vui_lm_config* c, const vui_lm_layer* layers, vui_lm_ctx* x, char* base);
+int sandwich_layers(vui_lm_ctx* x, const int64_t* tokens, int M, const LmRows& rows, hipStream_t st);

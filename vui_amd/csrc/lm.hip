@@ -6,30 +6,15 @@
 #include <string.h>
 
 #include <new>
-#include <vector>
 
 #include "lm.h"
 
-#define LM_EXPAND_FROM 64   // positions of one call from which keys and values are expanded per head
+#define LM_EXPAND_FROM 64  // positions of one call from which keys and values are expanded per head
+#define LM_ATTN_FROM 64    // ... from which sigmoid attention takes blocks of a prompt
+#define LM_GLA_FROM 5      // ... from which gated linear attention goes by chunks
 #define LM_MAX_SPLITS 64   // latent_value_kernel keeps one piece per lane
 
-static int pad(int v, int a) { return (v + a - 1) / a * a; }
-
-struct vui_lm_ctx {
-  vui_lm_config c;
-  vui_lm_weights w;
-  std::vector<vui_lm_layer> layers;
-  std::vector<vui_lm_dims> dims;
-  int R16;  // rows of the activation buffers
-  float* x; void* xt; float* ssq;
-  void *qu, *qr, *qlat;
-  float *craw, *gate, *part, *part_ml;
-  void* act;
-  float2* upd; void* sg; float2* agg;
-  void *kx, *vx;
-  float* layers_out;
-  int expand_from;
-};
+#define pad lm_pad
 
 static int lm_check_cfg(const vui_lm_config* c) {
   if (!c) { vui_set_error("config is NULL"); return VUI_EINVAL; }
@@ -38,10 +23,12 @@ static int lm_check_cfg(const vui_lm_config* c) {
     vui_set_error("lm: bad sizes width=%d vocab=%d layers=%d max_seqlen=%d slots=%d rows=%d", c->width, c->vocab, c->n_layers, c->max_seqlen, c->n_slots, c->max_rows);
     return VUI_EINVAL;
   }
+  if (c->norm_groups < 0 || (c->norm_groups > 0 && c->width % c->norm_groups)) {
+    vui_set_error("lm: a width of %d has no %d equal parts", c->width, c->norm_groups);
+    return VUI_EINVAL;
+  }
   return VUI_OK;
 }
-
-static size_t lm_esz(const vui_lm_config& c) { return c.dtype == VUI_DTYPE_F32 ? 4 : 2; }
 
 static bool lm_expands(const vui_lm_config& c, const vui_lm_dims& d) { return c.dtype == VUI_DTYPE_BF16 && latent_expand_ok(d); }
 
@@ -53,6 +40,7 @@ static int lm_splits(int M, int heads, int rank64) {
 }
 
 static size_t lm_carve(const vui_lm_config* c, const vui_lm_layer* layers, vui_lm_ctx* x, char* base) {
+  if (c->norm_groups > 0) return sandwich_carve(c, layers, x, base);
   const size_t e = lm_esz(*c);
   const size_t R = pad(c->max_rows < 16 ? 16 : c->max_rows, 16);
   size_t qu = 0, qr = 0, ql = 0, cr = 0, ga = 0, pt = 0, pm = 0, ac = 0, up = 0, kx = 0, vx = 0;
@@ -96,6 +84,7 @@ static size_t lm_carve(const vui_lm_config* c, const vui_lm_layer* layers, vui_l
 }
 
 static int lm_check_layer(const vui_lm_config& c, const vui_lm_layer& L, int l) {
+  if (c.norm_groups > 0) return sandwich_check_layer(c, L, l);
   if (L.ff < 0) { vui_set_error("layer %d: ff %d", l, L.ff); return VUI_EINVAL; }
   if (L.mixer == VUI_LM_MINGRU) {
     if (L.rnn_width < 1) { vui_set_error("layer %d: recurrence width %d", l, L.rnn_width); return VUI_EINVAL; }
@@ -116,6 +105,7 @@ int vui_lm_layer_dims(const vui_lm_config* c, const vui_lm_layer* L, vui_lm_dims
   if (!c || !L || !o) { vui_set_error("NULL argument"); return VUI_EINVAL; }
   memset(o, 0, sizeof(*o));
   o->w16 = pad(c->width, 16); o->w64 = pad(c->width, 64); o->s64 = pad(c->max_seqlen, 64);
+  if (c->norm_groups > 0) return sandwich_layer_dims(*c, *L, o);
   const bool attn = L->mixer == VUI_LM_LATENT_ATTENTION;
   const int tile = attn ? 32 : 48;  // rows of w_in a workgroup takes together
   int mix_k;
@@ -157,8 +147,10 @@ int vui_lm_create(const vui_lm_config* c, const vui_lm_layer* layers, const vui_
   if (!w->embed || !w->head || !w->final_norm) { vui_set_error("missing embedding, head or final norm"); return VUI_EINVAL; }
   for (int l = 0; l < c->n_layers; ++l) {
     const vui_lm_layer& L = layers[l];
-    bool ok = L.norm && L.w_in && L.w_out;
-    if (L.mixer == VUI_LM_MINGRU) {
+    bool ok = L.w_in && L.w_out && (c->norm_groups > 0 || L.norm);
+    if (c->norm_groups > 0) {
+      ok = ok && sandwich_pointers_ok(*c, L);
+    } else if (L.mixer == VUI_LM_MINGRU) {
       ok = ok && L.bias_z && L.bias_x && L.state;
     } else {
       ok = ok && L.w_uk_t && L.w_uv && L.c_cache && L.kr_cache && (L.rot_pairs == 0 || L.rope) && (L.kv_from >= 0 || L.latent_norm);
@@ -186,6 +178,8 @@ int vui_lm_create(const vui_lm_config* c, const vui_lm_layer* layers, const vui_
   x->R16 = pad(c->max_rows < 16 ? 16 : c->max_rows, 16);
   x->layers_out = nullptr;
   x->expand_from = LM_EXPAND_FROM;
+  x->attn_from = LM_ATTN_FROM;
+  x->gla_from = LM_GLA_FROM;
   lm_carve(c, layers, x, (char*)workspace);
   *out = x;
   return VUI_OK;
@@ -202,6 +196,13 @@ int vui_lm_debug_layers(vui_lm_ctx* ctx, float* buf) {
 int vui_lm_expand_from(vui_lm_ctx* ctx, int rows) {
   if (!ctx) { vui_set_error("NULL context"); return VUI_EINVAL; }
   ctx->expand_from = rows > 0 ? rows : LM_EXPAND_FROM;
+  return VUI_OK;
+}
+
+int vui_lm_block_from(vui_lm_ctx* ctx, int attn_rows, int gla_rows) {
+  if (!ctx) { vui_set_error("NULL context"); return VUI_EINVAL; }
+  ctx->attn_from = attn_rows > 0 ? attn_rows : LM_ATTN_FROM;
+  ctx->gla_from = gla_rows > 0 ? gla_rows : LM_GLA_FROM;
   return VUI_OK;
 }
 
@@ -265,6 +266,7 @@ static int lm_recurrence(vui_lm_ctx* x, int l, int M, const LmRows& rows, LmGemm
 
 static int lm_layers(vui_lm_ctx* x, const int64_t* tokens, int M, const LmRows& rows, hipStream_t st) {
   const vui_lm_config& c = x->c;
+  if (c.norm_groups > 0) return sandwich_layers(x, tokens, M, rows, st);
   const int w64 = x->dims[0].w64, np = x->dims[0].w16 / 16;
   int rc = launch_lm_embed(c.dtype, tokens, x->w.embed, x->x, x->xt, x->ssq, M, c.width, w64, np, c.vocab, st);
   if (rc) return rc;
@@ -315,7 +317,7 @@ int vui_lm_decode(vui_lm_ctx* x, const int64_t* tokens, const int32_t* slot_idx,
   if (rc) return rc;
   LmGemm g = lm_logits(x, r, B, B, nullptr, logits_out);
   g.upd_lens = seq_lens; g.upd_inc = seq_inc; g.upd_rows = B;
-  return launch_lm_gemm(x->c.dtype, LM_LOGITS, g, 1, st);
+  return launch_lm_gemm(x->c.dtype, x->c.norm_groups > 0 ? LM_HEAD : LM_LOGITS, g, 1, st);
 }
 
 int vui_lm_prefill(vui_lm_ctx* x, const int64_t* tokens, int T, int slot, int pos0, int32_t* seq_lens, const int32_t* want,
@@ -331,7 +333,7 @@ int vui_lm_prefill(vui_lm_ctx* x, const int64_t* tokens, int T, int slot, int po
   r.seq = 1; r.slot = slot; r.pos0 = pos0; r.S = x->c.max_seqlen; r.n_slots = x->c.n_slots;
   int rc = lm_layers(x, tokens, T, r, st);
   if (rc) return rc;
-  if (n_want > 0 && (rc = launch_lm_gemm(x->c.dtype, LM_LOGITS, lm_logits(x, r, n_want, T, want, logits_out), 1, st))) return rc;
+  if (n_want > 0 && (rc = launch_lm_gemm(x->c.dtype, x->c.norm_groups > 0 ? LM_HEAD : LM_LOGITS, lm_logits(x, r, n_want, T, want, logits_out), 1, st))) return rc;
   hipLaunchKernelGGL(lm_set_len_kernel, dim3(1), dim3(1), 0, st, seq_lens, slot, pos0 + T);
   HIP_TRY(hipGetLastError());
   return VUI_OK;

@@ -2,7 +2,7 @@
 // matrix cores (bf16 or true fp32), both operands tiled, K split over the waves of a workgroup (partial tiles meet in
 // LDS and are added in wave order).  What a layer does with the sums is the epilogue.
 //
-// The layers' norm has a single number for its weight, so W norm(x) = s W x with one scale s per row: the product
+// Parallel layers: the norm has a single number for its weight, so W norm(x) = s W x with one scale s per row: the product
 // runs on the raw residual row and the epilogue scales.  The sum of squares behind s is left by whoever wrote the
 // row, in pieces of 16 columns (LM_OUT, the embedding), so no launch is spent on norms.
 #include "common.h"
@@ -31,18 +31,32 @@ __device__ __forceinline__ void lm_rotate2(float* v, const float* rope, int pos,
   }
 }
 
+// activations of ungated feed-forwards
+__device__ __forceinline__ float lm_act(float z, int kind, float pos, float neg) {
+  if (kind == VUI_LM_ACT_RELU2) { z = fmaxf(z, 0.f); return z * z; }
+  const float m = fminf(z, 0.f);
+  return (z > 0.f ? pos * z * z : neg * (expm1f(m) - m)) + 0.5f * z;
+}
+
 template <typename T, int MB, int NB, int WAVES, int EPI>
 __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
   constexpr bool SCALED = EPI == LM_IN_ATTN || EPI == LM_IN_GRU_STEP || EPI == LM_IN_GRU_SEQ || EPI == LM_LOGITS;
   constexpr bool GRU = EPI == LM_IN_GRU_STEP || EPI == LM_IN_GRU_SEQ;
+  constexpr bool LOGITS = EPI == LM_LOGITS || EPI == LM_HEAD, MOE = EPI == LM_MOE_UP || EPI == LM_MOE_DOWN;
   constexpr bool ROWS_FIRST = EPI == LM_EXPAND_V;  // a lane then holds four consecutive rows of one feature
   constexpr int EP = Tl<T>::EP, P = 16 / EP, TILE = MB * NB * 256;
   __shared__ __align__(16) float part[WAVES * TILE];
   __shared__ float srow[MB * 16];
   const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63;
   const int l16 = lane & 15, kg = lane >> 4;
-  const int MT = (p.M + 16 * MB - 1) / (16 * MB);
+  const int MT = MOE ? p.max_tiles : (p.M + 16 * MB - 1) / (16 * MB);
   const int m0 = ((int)blockIdx.x % MT) * 16 * MB, nb0 = ((int)blockIdx.x / MT) * NB;
+  size_t wz = blockIdx.z * p.wz;
+  if (MOE) {
+    const int t = (int)blockIdx.x % MT;
+    if (t >= p.n_tiles[0]) return;  // uniform
+    wz = (size_t)p.tile_e[t] * p.wz;
+  }
   const int nsteps = p.K >> 6;
   const int s0 = nsteps * wave / WAVES, s1 = nsteps * (wave + 1) / WAVES;
   const int MBL = (p.M + 15) >> 4, NBL = p.N >> 4;
@@ -51,7 +65,12 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
   const T* wr[NB];
 #pragma unroll
   for (int j = 0; j < MB; ++j) {
-    if (EPI == LM_LOGITS && p.rowmap) {
+    if (EPI == LM_MOE_UP) {
+      const int e = p.ent[m0 + 16 * j + l16], r = min(max(e, 0) / p.top, p.x_rows - 1);
+      xr[j] = (const T*)p.X + (size_t)(r >> 4) * nsteps * 1024 + ((r & 15) + 16 * kg) * EP;
+    } else if (EPI == LM_MOE_DOWN) {
+      xr[j] = (const T*)p.X + (size_t)((m0 >> 4) + j) * nsteps * 1024 + lane * EP;
+    } else if (LOGITS && p.rowmap) {
       const int r = min(max(p.rowmap[min(m0 + 16 * j + l16, p.M - 1)], 0), p.x_rows - 1);
       xr[j] = (const T*)p.X + (size_t)(r >> 4) * nsteps * 1024 + ((r & 15) + 16 * kg) * EP;
     } else {
@@ -62,7 +81,7 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
   }
 #pragma unroll
   for (int i = 0; i < NB; ++i)
-    wr[i] = (const T*)p.W + blockIdx.z * p.wz + (size_t)min(nb0 + i, NBL - 1) * nsteps * 1024 + lane * EP;
+    wr[i] = (const T*)p.W + wz + (size_t)min(nb0 + i, NBL - 1) * nsteps * 1024 + lane * EP;
 
   // What the scale and the epilogue of this wave's first unit will need is requested now, ahead of the operands:
   // fetched where it is used, it would be a chain of dependent loads behind the last product.
@@ -73,7 +92,7 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
   float sq[NSQ], norm = 0.f;
   if (SCALED) {
     sq_m = min(m0 + min(sq_r, MB * 16 - 1), p.M - 1);
-    if (EPI == LM_LOGITS && p.rowmap) sq_m = min(max(p.rowmap[sq_m], 0), p.x_rows - 1);
+    if (LOGITS && p.rowmap) sq_m = min(max(p.rowmap[sq_m], 0), p.x_rows - 1);
 #pragma unroll
     for (int i = 0; i < NSQ; ++i) sq[i] = p.ssq[(size_t)sq_m * p.np + min(sq_q + TPR * i, p.np - 1)];
     norm = p.norm[0];
@@ -150,7 +169,7 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
     const int m = m0 + 16 * j + (ROWS_FIRST ? 4 * kg : l16);
     const int nb = nb0 + i0;
     const int n = nb * 16 + (ROWS_FIRST ? l16 : 4 * kg);
-    const bool live = m < p.M && nb < NBL;
+    const bool live = (MOE || m < p.M) && nb < NBL;
     const float sc = SCALED ? srow[16 * j + l16] : 1.f;
     float v[4];
     auto gather = [&](int i, float* o) {
@@ -247,9 +266,27 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
       if (live && kg == 0 && nb < p.np) p.ssq_out[(size_t)m * p.np + nb] = sq;
       continue;
     }
-    if (EPI == LM_LOGITS) {
+    if (LOGITS) {
       if (live)
         for (int r = 0; r < 4; ++r) if (n + r < p.vocab) p.logits[(size_t)m * p.vocab + n + r] = v[r];
+      continue;
+    }
+    if (EPI == LM_PROJ || EPI == LM_PLAIN || EPI == LM_MOE_DOWN) {
+      const int r = EPI == LM_MOE_DOWN ? p.ent[m] : m;
+      if (!live || r < 0) continue;
+      if (EPI != LM_MOE_DOWN && p.bias) {
+        const float4 b = *reinterpret_cast<const float4*>(p.bias + n);
+        v[0] += b.x; v[1] += b.y; v[2] += b.z; v[3] += b.w;
+      }
+      if (EPI == LM_PROJ) Tl<T>::st4((T*)p.out + (size_t)r * p.ldo + n, v);
+      else Tl<float>::st4((float*)p.out + (size_t)r * p.ldo + n, v);
+      continue;
+    }
+    if (EPI == LM_ACT || EPI == LM_MOE_UP) {
+      if (!live) continue;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) v[r] = lm_act(v[r], p.act_kind, p.act_pos, p.act_neg);
+      Tl<T>::st4((T*)p.act + tl_off<T>(m, n, p.act_k), v);
       continue;
     }
     if (EPI == LM_EXPAND_K) {
@@ -266,7 +303,7 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
       continue;
     }
   }
-  if (EPI == LM_LOGITS && p.upd_lens && blockIdx.x == 0) {
+  if (LOGITS && p.upd_lens && blockIdx.x == 0) {
     if (p.upd_inc) {
       for (int s = tid; s < p.rows.n_slots; s += 64 * WAVES) p.upd_lens[s] += p.upd_inc[s];
     } else {
@@ -277,7 +314,8 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
 
 template <typename T, int MB, int NB, int WAVES, int EPI>
 static int go(const LmGemm& g, int nz, hipStream_t st) {
-  const int tiles = ((g.M + 16 * MB - 1) / (16 * MB)) * ((g.N / 16 + NB - 1) / NB);
+  const bool moe = EPI == LM_MOE_UP || EPI == LM_MOE_DOWN;
+  const int tiles = (moe ? g.max_tiles : (g.M + 16 * MB - 1) / (16 * MB)) * ((g.N / 16 + NB - 1) / NB);
   hipLaunchKernelGGL((lm_gemm_kernel<T, MB, NB, WAVES, EPI>), dim3((unsigned)tiles, 1, nz), dim3(64 * WAVES), 0, st, g);
   HIP_TRY(hipGetLastError());
   return VUI_OK;
@@ -293,6 +331,12 @@ static int pick(int epi, const LmGemm& g, int nz, hipStream_t st) {
     case LM_IN_GRU_SEQ: return few ? go<T, 1, 3, 8, LM_IN_GRU_SEQ>(g, nz, st) : go<T, 2, 3, 4, LM_IN_GRU_SEQ>(g, nz, st);
     case LM_OUT: return few ? go<T, 1, 1, 16, LM_OUT>(g, nz, st) : go<T, 2, 2, 4, LM_OUT>(g, nz, st);
     case LM_LOGITS: return few ? go<T, 1, 2, 8, LM_LOGITS>(g, nz, st) : go<T, 2, 2, 4, LM_LOGITS>(g, nz, st);
+    case LM_HEAD: return few ? go<T, 1, 2, 8, LM_HEAD>(g, nz, st) : go<T, 2, 2, 4, LM_HEAD>(g, nz, st);
+    case LM_PROJ: return few ? go<T, 1, 2, 8, LM_PROJ>(g, nz, st) : go<T, 2, 2, 4, LM_PROJ>(g, nz, st);
+    case LM_PLAIN: return few ? go<T, 1, 1, 16, LM_PLAIN>(g, nz, st) : go<T, 2, 2, 4, LM_PLAIN>(g, nz, st);
+    case LM_ACT: return few ? go<T, 1, 2, 8, LM_ACT>(g, nz, st) : go<T, 2, 2, 4, LM_ACT>(g, nz, st);
+    case LM_MOE_UP: return few ? go<T, 1, 2, 8, LM_MOE_UP>(g, nz, st) : go<T, 2, 2, 4, LM_MOE_UP>(g, nz, st);
+    case LM_MOE_DOWN: return few ? go<T, 1, 2, 8, LM_MOE_DOWN>(g, nz, st) : go<T, 2, 2, 4, LM_MOE_DOWN>(g, nz, st);
     case LM_EXPAND_K: return go<T, 2, 2, 4, LM_EXPAND_K>(g, nz, st);
     case LM_EXPAND_V: return go<T, 2, 2, 4, LM_EXPAND_V>(g, nz, st);
   }

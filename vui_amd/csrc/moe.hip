@@ -1,0 +1,91 @@
+// Expert routing: the `top` largest router logits of a row (the lower index wins a tie), shares by softmax over those, and
+// the (row, choice) entries sorted by expert, every expert's padded to whole tiles of the products that follow.
+#include "common.h"
+#include "lm.h"
+
+// one wave; picks in order of falling logits, so "behind the last pick" needs no list of what was taken
+__device__ __forceinline__ void route_row(const RouteArgs& p, int m) {
+  const int lane = threadIdx.x & 63;
+  const float* z = p.logits + (size_t)m * p.ldl;
+  float last = INFINITY, vmax = 0.f, sum = 0.f, mine = 0.f;
+  int last_e = -1;
+  for (int c = 0; c < p.top; ++c) {
+    float bv = -INFINITY;
+    int be = 0x7fffffff;
+    for (int e = lane; e < p.E; e += 64) {
+      const float v = z[e];
+      if ((v < last || (v == last && e > last_e)) && (v > bv || be == 0x7fffffff)) { bv = v; be = e; }
+    }
+#pragma unroll
+    for (int o = 32; o >= 1; o >>= 1) {
+      const float ov = __shfl_xor(bv, o);
+      const int oe = __shfl_xor(be, o);
+      if (oe != 0x7fffffff && (be == 0x7fffffff || ov > bv || (ov == bv && oe < be))) { bv = ov; be = oe; }
+    }
+    if (c == 0) vmax = bv;
+    const float w = expf(bv - vmax);
+    sum += w;
+    if (lane == c) mine = w;
+    if (lane == 0) p.choice[(size_t)m * p.top + c] = be < p.E ? be : 0;
+    last = bv;
+    last_e = be;
+  }
+  if (lane < p.top) p.share[(size_t)m * p.top + lane] = mine / sum;
+}
+
+__global__ __launch_bounds__(256) void moe_top_kernel(const RouteArgs p) {
+  const int m = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (m < p.M) route_row(p, m);
+}
+
+// One workgroup sorts all entries.  Where an entry lands inside its expert's run has no effect on its numbers.
+template <bool TOP>
+__global__ __launch_bounds__(1024) void moe_sort_kernel(const RouteArgs p) {
+  __shared__ int cnt[VUI_LM_MAX_EXPERTS], start[VUI_LM_MAX_EXPERTS], wsum[16];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, n = p.M * p.top;
+  cnt[tid] = 0;
+  if (TOP) {
+    for (int m = wave; m < p.M; m += 16) route_row(p, m);
+    __threadfence_block();
+  }
+  __syncthreads();
+  for (int i = tid; i < n; i += 1024) atomicAdd(&cnt[p.choice[i]], 1);
+  __syncthreads();
+  const int tiles = tid < p.E ? (cnt[tid] + p.tile_rows - 1) / p.tile_rows : 0;
+  int s = tiles;  // inclusive sum over the wave
+#pragma unroll
+  for (int o = 1; o < 64; o <<= 1) {
+    const int v = __shfl_up(s, o);
+    if (lane >= o) s += v;
+  }
+  if (lane == 63) wsum[wave] = s;
+  __syncthreads();
+  for (int w = 0; w < wave; ++w) s += wsum[w];
+  const int first = s - tiles;
+  for (int t = first; t < s; ++t) p.tile_e[t] = tid;
+  for (int i = first * p.tile_rows + (tid < p.E ? cnt[tid] : 0); i < s * p.tile_rows; ++i) p.ent[i] = -1;
+  start[tid] = first * p.tile_rows;
+  if (tid == 1023) p.n_tiles[0] = s;
+  __syncthreads();
+  cnt[tid] = 0;
+  __syncthreads();
+  for (int i = tid; i < n; i += 1024) {
+    const int e = p.choice[i];
+    p.ent[start[e] + atomicAdd(&cnt[e], 1)] = i;
+  }
+}
+
+int launch_moe_route(const RouteArgs& a, hipStream_t st) {
+  if (a.M < 1 || a.E < 1 || a.E > VUI_LM_MAX_EXPERTS || a.top < 1 || a.top > VUI_LM_MAX_TOP || a.top > a.E || a.ldl < a.E) {
+    vui_set_error("expert routing: bad shape M=%d experts=%d top=%d", a.M, a.E, a.top);
+    return VUI_EINVAL;
+  }
+  if (a.M <= 16) {
+    hipLaunchKernelGGL(moe_sort_kernel<true>, dim3(1), dim3(1024), 0, st, a);
+  } else {
+    hipLaunchKernelGGL(moe_top_kernel, dim3((a.M + 3) / 4), dim3(256), 0, st, a);
+    hipLaunchKernelGGL(moe_sort_kernel<false>, dim3(1), dim3(1024), 0, st, a);
+  }
+  HIP_TRY(hipGetLastError());
+  return VUI_OK;
+}
