@@ -117,7 +117,7 @@ def distance_bucket(n: int, buckets: int, far: int) -> int:
     half = buckets // 2
     if n < half:
         return n
-    if far <= half:
+    if half < 1 or far <= half:
         return buckets - 1
     return min(buckets - 1, half + math.floor(math.log(n / half) / math.log(far / half) * (buckets - half) + 1e-9))
 
@@ -154,8 +154,9 @@ def xielu_mlp(h: Tensor, w: dict, p: str) -> Tensor:
     return xielu(h @ w[p + "up"].T, *w[p + "act"]) @ w[p + "down"].T
 
 
-def expert_mlp(h: Tensor, w: dict, p: str, router: dict) -> Tensor:
-    """The `top` experts with the largest router logits per token, weighed by a softmax over those; relu squared inside."""
+def expert_mlp(h: Tensor, w: dict, p: str, router: dict, margins: "list | None" = None) -> Tensor:
+    """The `top` experts with the largest router logits per token, weighed by a softmax over those; relu squared inside.
+    margins, if given, receives how far every token was from another choice (T)."""
     z = h @ w[p + "router"].T + w[p + "router.b"]
     out = torch.zeros_like(h)
     for t in range(len(h)):
@@ -163,6 +164,9 @@ def expert_mlp(h: Tensor, w: dict, p: str, router: dict) -> Tensor:
         share = torch.softmax(best.values, 0)
         for e, s in zip(best.indices.tolist(), share):
             out[t] += s * (torch.relu(h[t] @ w[f"{p}e{e}.up"].T).square() @ w[f"{p}e{e}.down"].T)
+    if margins is not None:
+        v = torch.sort(z, dim=1, descending=True).values
+        margins.append(v[:, router["top"] - 1] - v[:, router["top"]] if router["top"] < v.shape[1] else torch.full_like(v[:, 0], math.inf))
     return out
 
 
@@ -177,7 +181,7 @@ def layer_passes(cfg: dict) -> "list[tuple[int, int | None]]":
     return order + [(i, None) for i in range(loop["stop"], n)]
 
 
-def forward_sandwich(cfg: dict, w: dict, tokens, layers_out: "list | None" = None) -> Tensor:
+def forward_sandwich(cfg: dict, w: dict, tokens, layers_out: "list | None" = None, margins: "list | None" = None) -> Tensor:
     """Mabidra: norms on both sides of every sublayer, a loop over some layers that mixes the embedding back in."""
     eps, groups = cfg["norm"]["eps"], cfg["norm"]["groups"]
     x = x0 = w["embed"][torch.as_tensor(tokens, dtype=torch.long)] * cfg["embedding"]["scale"]
@@ -197,18 +201,18 @@ def forward_sandwich(cfg: dict, w: dict, tokens, layers_out: "list | None" = Non
         mlp = layer.get("mlp")
         if mlp is not None:
             h = grouped_norm(x, w[p + "norm2"], groups, eps)
-            y = xielu_mlp(h, w, p + "mlp.") if mlp["kind"] == "dense" else expert_mlp(h, w, p + "mlp.", mlp["router"])
+            y = xielu_mlp(h, w, p + "mlp.") if mlp["kind"] == "dense" else expert_mlp(h, w, p + "mlp.", mlp["router"], margins)
             x = x + grouped_norm(y, w[p + "norm2b"], groups, eps)
         if layers_out is not None:
             layers_out.append(x.clone())
     return grouped_norm(x, w["final.norm"], groups, eps) @ w["head"].T
 
 
-def forward(cfg: dict, w: dict, tokens, dtype=torch.float64, layers_out: "list | None" = None) -> Tensor:
-    """Logits (T, vocab) of one sequence.  layers_out, if given, receives the residual stream behind each layer."""
+def forward(cfg: dict, w: dict, tokens, dtype=torch.float64, layers_out: "list | None" = None, margins: "list | None" = None) -> Tensor:
+    """Logits (T, vocab) of one sequence.  layers_out, if given, receives the residual stream behind each layer run."""
     w = {k: v.to(dtype) for k, v in w.items()}
     if cfg["architecture"] == "Mabidra":
-        return forward_sandwich(cfg, w, tokens, layers_out)
+        return forward_sandwich(cfg, w, tokens, layers_out, margins)
     eps = cfg["norm"]["eps"]
     x = w["embed"][torch.as_tensor(tokens, dtype=torch.long)]
     entries: dict = {}

@@ -148,7 +148,7 @@ def distance_buckets(n: int, buckets: int, far: int) -> "list[int]":
     for d in range(n):
         if d < half:
             out.append(d)
-        elif far <= half:
+        elif half < 1 or far <= half:
             out.append(buckets - 1)
         else:
             steps = buckets - half
