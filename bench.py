@@ -520,14 +520,38 @@ LM_SIZES = [("w768", 768, 8, 2048, 64, 32, 96, 256, 8), ("w1024", 1024, 8, 2816,
             ("w2048", 2048, 16, 4096, 128, 64, 128, 512, 8)]
 
 
+# Sizes of the lines of sandwich layers: (name, width, heads, key groups, dim, ff, layers).  The token model beside each is
+# the one above of that name; two matrices instead of three make the feed-forward, hence 1.5 times its features.
+SANDWICH_SIZES = [("w768", 768, 8, 2, 96, 3072, 8), ("w1024", 1024, 8, 2, 128, 4224, 8), ("w2048", 2048, 16, 4, 128, 6144, 8)]
+
+
 def lm_work(cfg, L: float, B: int):
     """(bytes of one decode step of B rows at cache length L, flops of its weights per token, flops of attention per
-    token and visible key in the expanded form).  Every weight, latent, key part and state once, bf16."""
+    token and visible key in the expanded form).  Every weight, latent, key part and state once, bf16; of an expert
+    layer the experts that B tokens reach on average."""
     W = cfg["width"]
     wb = W * cfg["vocab"]
-    cache = state = attn = 0
+    cache = state = attn = idle = 0
     for layer in cfg["layers"]:
-        mx = layer["mixer"]
+        mx, mlp = layer["mixer"], layer["mlp"]
+        if layer["type"] in ("gla", "attention"):
+            H, dk, dv = mx["heads"], mx["dim"], mx["vdim"]
+            if layer["type"] == "gla":
+                r = cfg.get("gla_rank", 16)
+                wb += W * (2 * H * (dk + dv) + r) + H * dk * r + W * H * dv
+                state += 8 * H * dk * dv
+            else:
+                G = mx["kv_heads"]
+                wb += W * (H * dk + G * (dk + dv) + H) + W * H * dv
+                cache += 2 * G * (dk + dv)
+                attn += 2 * H * (dk + dv)
+            if mlp["kind"] == "moe":
+                n, top, f = mlp["router"]["experts"], mlp["router"]["top"], mlp["expert"]["ff"]
+                wb += W * n + 2 * W * f * top
+                idle += 2 * W * f * (n * (1 - (1 - top / n) ** B) - top)  # weights read for other rows of the batch
+            else:
+                wb += 2 * W * mlp["ff"]
+            continue
         if layer["type"] == "latent_attention":
             H, r = mx["heads"], mx["kv_rank"]
             wb += W * (H * (mx["dim"] + mx["rot_dim"]) + (0 if "kv_from" in mx else r + mx["rot_dim"]) + H + H * mx["vdim"]) + H * r * (mx["dim"] + mx["vdim"])
@@ -537,7 +561,77 @@ def lm_work(cfg, L: float, B: int):
             wb += 4 * W * mx["width"]
             state += 8 * mx["width"]
         wb += 3 * W * layer["mlp"]["ff"]
-    return wb * 2 + B * (cache * L + state), 2 * (wb - W * cfg["vocab"]), attn
+    if cfg.get("loop"):
+        wb += 2 * W * W
+    return (wb + idle) * 2 + B * (cache * L + state), 2 * (wb - W * cfg["vocab"]), attn
+
+
+def event_us(fn, n):
+    """Microseconds of one call, from events around n of them."""
+    import torch
+
+    fn()
+    torch.cuda.synchronize()
+    e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+    e0.record()
+    for _ in range(n):
+        fn()
+    e1.record()
+    torch.cuda.synchronize()
+    return e0.elapsed_time(e1) * 1e3 / n
+
+
+def token_model_line(cfg, batches, prompts, L, S):
+    """Prefill of one prompt and the captured decode step of B rows at cache length L of a token model with random weights."""
+    import torch
+
+    from vui_amd.lm import TokenLM
+    from vui_amd.lm_engine import TokenEngine
+    from vui_amd.synthetic import token_lm_state_dict
+
+    out = {}
+    eng = TokenEngine(model=TokenLM.from_config(cfg, token_lm_state_dict(cfg, 0, "cuda"), max_seqlen=S), max_rows=16)
+    m = eng.model
+    for group in (m.cache.c, m.cache.kr, m.cache.k, m.cache.v):
+        for t in group.values():
+            t.normal_()
+    toks = torch.randint(0, cfg["vocab"], (S,), device="cuda")
+    for T in prompts:
+        us = event_us(lambda: m.prefill(toks[:T], 0, 0, [T - 1]), 5)
+        _, fl, at = lm_work(cfg, 0, 1)
+        fl = fl * T + at * T * (T + 1) / 2
+        out[f"prefill_{T}"] = {"ms": round(us / 1e3, 3), "tokens_per_s": round(T * 1e6 / us), "TFLOPs": round(fl / us / 1e6, 1), "mfma_frac": round(fl / us / 1e6 / 2500, 4)}
+    for B in batches:
+        eng._set_active_slots(list(range(B)))
+        eng.seq_lens.fill_(L - 26)
+        eng._g_tokens[:B] = toks[:B]
+        us = event_us(lambda: eng._replay_bucket(B, eng._decode_body), 50)
+        by, _, _ = lm_work(cfg, L, B)
+        out[f"decode_b{B}"] = {"us": round(us, 1), "tokens_per_s": round(B * 1e6 / us), "GBs": round(by / us / 1e3, 1), "hbm_frac": round(by / us / 1e3 / HBM_PEAK_GBS, 4)}
+    return out
+
+
+def sandwich_lines(sizes=None, batches=(1, 4, 16), prompts=(512, 2048), L=1024, which="both"):
+    """Token models of sandwich layers (Mabidra) beside the token model of parallel layers (Sakupel) of equal size."""
+    import torch
+
+    from vui_amd.synthetic import sandwich_lm_config, token_lm_config
+
+    S = max(2304, L + 256, max(prompts, default=0) + 16)
+    like = {size[0]: size[1:] for size in LM_SIZES}
+    for name, W, H, G, dim, F, nl in SANDWICH_SIZES:
+        if sizes and name not in sizes:
+            continue
+        out = {"config": f"sandwich_lm_{name}", "dtype": "bf16", "data": "synthetic", "layers": nl, "width": W, "heads": H, "kv_heads": G,
+               "dim": dim, "ff": F, "experts": 32, "top": 4}
+        if which in ("both", "lm"):
+            out.update(token_model_line(sandwich_lm_config(W, H, G, dim, F, 32, 4, nl, vocab=2048), batches, prompts, L, S))
+        torch.cuda.empty_cache()
+        if which in ("both", "like"):
+            lW, lH, lF, ldim, lrot, lvdim, lrank, lnl = like[name]
+            out["parallel_layers"] = token_model_line(token_lm_config(lW, lH, lF, ldim, lrot, lvdim, lrank, lnl, vocab=2048), batches, prompts, L, S)
+        torch.cuda.empty_cache()
+        yield out
 
 
 def lm_lines(sizes=None, batches=(1, 4, 16), prompts=(512, 2048), L=1024, which="both"):
@@ -548,21 +642,8 @@ def lm_lines(sizes=None, batches=(1, 4, 16), prompts=(512, 2048), L=1024, which=
 
     from vui_amd.config import Config, DataConfig, VuiConfig
     from vui_amd.engine import Engine
-    from vui_amd.lm import TokenLM
-    from vui_amd.lm_engine import TokenEngine
     from vui_amd.model import Vui
-    from vui_amd.synthetic import synthetic_state_dict, token_lm_config, token_lm_state_dict
-
-    def timed(fn, n):
-        fn()
-        torch.cuda.synchronize()
-        e0, e1 = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
-        e0.record()
-        for _ in range(n):
-            fn()
-        e1.record()
-        torch.cuda.synchronize()
-        return e0.elapsed_time(e1) * 1e3 / n
+    from vui_amd.synthetic import synthetic_state_dict, token_lm_config
 
     S = max(2304, L + 256, max(prompts, default=0) + 16)
     for name, W, H, F, dim, rot, vdim, rank, nl in LM_SIZES:
@@ -570,27 +651,7 @@ def lm_lines(sizes=None, batches=(1, 4, 16), prompts=(512, 2048), L=1024, which=
             continue
         out = {"config": f"token_lm_{name}", "dtype": "bf16", "data": "synthetic", "layers": nl, "width": W, "heads": H, "ff": F, "kv_rank": rank}
         if which in ("both", "lm"):
-            cfg = token_lm_config(W, H, F, dim, rot, vdim, rank, nl, vocab=2048)
-            eng = TokenEngine(model=TokenLM.from_config(cfg, token_lm_state_dict(cfg, 0, "cuda"), max_seqlen=S), max_rows=16)
-            m = eng.model
-            for t in m.cache.c.values():
-                t.normal_()
-            for t in m.cache.kr.values():
-                t.normal_()
-            toks = torch.randint(0, cfg["vocab"], (S,), device="cuda")
-            for T in prompts:
-                us = timed(lambda: m.prefill(toks[:T], 0, 0, [T - 1]), 5)
-                _, fl, at = lm_work(cfg, 0, 1)
-                fl = fl * T + at * T * (T + 1) / 2
-                out[f"prefill_{T}"] = {"ms": round(us / 1e3, 3), "tokens_per_s": round(T * 1e6 / us), "TFLOPs": round(fl / us / 1e6, 1), "mfma_frac": round(fl / us / 1e6 / 2500, 4)}
-            for B in batches:
-                eng._set_active_slots(list(range(B)))
-                eng.seq_lens.fill_(L - 26)
-                eng._g_tokens[:B] = toks[:B]
-                us = timed(lambda: eng._replay_bucket(B, eng._decode_body), 50)
-                by, _, _ = lm_work(cfg, L, B)
-                out[f"decode_b{B}"] = {"us": round(us, 1), "tokens_per_s": round(B * 1e6 / us), "GBs": round(by / us / 1e3, 1), "hbm_frac": round(by / us / 1e3 / HBM_PEAK_GBS, 4)}
-            del eng, m
+            out.update(token_model_line(token_lm_config(W, H, F, dim, rot, vdim, rank, nl, vocab=2048), batches, prompts, L, S))
         if which in ("both", "vui"):
             c = VuiConfig(d_model=W, n_layers=nl, n_heads=H, intermediate_size=F, n_quantizers=16, codebook_size=2048, use_rq_transformer=True,
                           rq_d_model=512, rq_n_layers=4, rq_n_heads=8, vocab_size=512, max_text_tokens=S - 16, max_audio_tokens=0)
@@ -603,7 +664,7 @@ def lm_lines(sizes=None, batches=(1, 4, 16), prompts=(512, 2048), L=1024, which=
                 vm.decoder._v.normal_()
                 ve._decode_step()
                 ve.seq_lens.fill_(L - 26)
-                us = timed(ve._decode_graph.replay, 50)
+                us = event_us(ve._decode_graph.replay, 50)
                 vm._native.status()
                 by = (wl + W * 2048) * 2 + B * L * nl * 4 * W
                 vui[f"decode_b{B}"] = {"us": round(us, 1), "tokens_per_s": round(B * 1e6 / us), "GBs": round(by / us / 1e3, 1), "hbm_frac": round(by / us / 1e3 / HBM_PEAK_GBS, 4)}
@@ -614,7 +675,7 @@ def lm_lines(sizes=None, batches=(1, 4, 16), prompts=(512, 2048), L=1024, which=
                         def pre():
                             ve.seq_lens[0] = 0
                             vm.decoder.forward_flash(emb[:, :T], None, slot_idx=None, known=(0, 0))
-                        us = timed(pre, 5)
+                        us = event_us(pre, 5)
                         fl = 2 * wl * T + nl * 4 * W * T * (T + 1) / 2
                         vui[f"prefill_{T}"] = {"ms": round(us / 1e3, 3), "tokens_per_s": round(T * 1e6 / us), "TFLOPs": round(fl / us / 1e6, 1), "mfma_frac": round(fl / us / 1e6 / 2500, 4)}
                 del ve
@@ -860,10 +921,13 @@ def main():
                     help="print only the streamed turn with audio on a divided GPU (the run its rocprofv3 summary comes from)")
     ap.add_argument("--lm", nargs="*", metavar="SIZE", default=None,
                     help="print only the token-model lines (sizes: w768 w1024 w2048; none named: all), each beside the Vui backbone of equal size")
-    ap.add_argument("--lm-which", default="both", choices=["both", "lm", "vui"], help="one side of the --lm lines (for profiles)")
-    ap.add_argument("--lm-batch", type=int, nargs="*", default=[1, 4, 16], help="rows of the --lm decode steps")
-    ap.add_argument("--lm-prompt", type=int, nargs="*", default=[512, 2048], help="prompt lengths of the --lm lines")
-    ap.add_argument("--lm-length", type=int, default=1024, help="cache length of the --lm decode steps")
+    ap.add_argument("--sandwich-lm", nargs="*", metavar="SIZE", default=None,
+                    help="print only the lines of token models with sandwich layers, each beside the --lm model of that size")
+    ap.add_argument("--lm-which", default="both", choices=["both", "lm", "vui", "like"],
+                    help="one side of the lines (for profiles): the model itself, or what is beside it (--lm: vui, --sandwich-lm: like)")
+    ap.add_argument("--lm-batch", type=int, nargs="*", default=[1, 4, 16], help="rows of the token-model decode steps")
+    ap.add_argument("--lm-prompt", type=int, nargs="*", default=[512, 2048], help="prompt lengths of the token-model lines")
+    ap.add_argument("--lm-length", type=int, default=1024, help="cache length of the token-model decode steps")
     ap.add_argument("--phase-clock", action="store_true",
                     help="print the phase stamps of one workgroup of the batch-1 frame kernel (with --int8: int8 weights)")
     ap.add_argument("--bb-phase-clock", type=int, default=0, metavar="ROWS",
@@ -878,6 +942,10 @@ def main():
         sys.exit(2)
     if args.lm is not None:
         for ln in lm_lines(args.lm, args.lm_batch, args.lm_prompt, L=args.lm_length, which=args.lm_which):
+            print(json.dumps(ln), flush=True)
+        return
+    if args.sandwich_lm is not None:
+        for ln in sandwich_lines(args.sandwich_lm, args.lm_batch, args.lm_prompt, L=args.lm_length, which=args.lm_which):
             print(json.dumps(ln), flush=True)
         return
     if args.phase_clock:

@@ -132,8 +132,28 @@ def token_lm_config(width: int, heads: int, ff: int, dim: int, rot_dim: int, vdi
     return {"architecture": "Sakupel", "width": width, "vocab": vocab, "norm": {"eps": 1e-5}, "layers": layers}
 
 
+def sandwich_lm_config(width: int, heads: int, kv_heads: int, dim: int, ff: int, experts: int, top: int, n_layers: int,
+                       vocab: int = 8192, rank: int = 32) -> dict:
+    """A Mabidra configuration whose layers repeat the pattern: gated linear attention, attention, attention, attention;
+    every second feed-forward is made of experts, `top` of which have the ff features of a dense one together.  One
+    pass over all layers (a loop of one time, so that its mixing product is there)."""
+    layers = []
+    for i in range(n_layers):
+        mlp = {"kind": "dense", "ff": ff} if i % 2 == 0 else {
+            "kind": "moe", "expert": {"ff": ff // top}, "router": {"experts": experts, "top": top}}
+        if i % 4 == 0:
+            layers.append({"type": "gla", "mixer": {"heads": heads // 2, "dim": dim, "vdim": 2 * dim, "tau": 8.0}, "mlp": mlp})
+            continue
+        layers.append({"type": "attention", "mlp": mlp, "mixer": {
+            "heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "bias_max": 1000,
+            "q_temp": {"coef": 0.1, "every": 500}}})
+    return {"architecture": "Mabidra", "width": width, "vocab": vocab, "norm": {"eps": 1e-5, "groups": 4}, "layers": layers,
+            "embedding": {"scale": 1.0}, "loop": {"start": 0, "stop": n_layers, "times": 1}, "gla_rank": rank}
+
+
 def token_lm_state_dict(cfg: dict, seed: int = 0, device="cpu") -> dict[str, Tensor]:
-    """Random bf16 weights N(0, 1 / fan_in) of a token model's configuration, norm weights 1, biases 0."""
+    """Random bf16 weights N(0, 1 / fan_in) of a token model's configuration, norm weights 1, biases 0 (`gla_rank`: rank of
+    the decays of gated linear attention, which a checkpoint tells by a shape)."""
     g = torch.Generator(device=device).manual_seed(seed)
     W = cfg["width"]
     sd: dict[str, Tensor] = {}
@@ -144,9 +164,52 @@ def token_lm_state_dict(cfg: dict, seed: int = 0, device="cpu") -> dict[str, Ten
     def ones(name: str, *shape: int) -> None:
         sd[name] = torch.ones(shape, dtype=torch.bfloat16, device=device)
 
+    def zeros(name: str, *shape: int) -> None:
+        sd[name] = torch.zeros(shape, dtype=torch.bfloat16, device=device)
+
+    sandwich = cfg["architecture"] == "Mabidra"
     mat("embed", cfg["vocab"], W)
+    if cfg.get("loop"):
+        mat("loop.in", W, 2 * W)
+        zeros("loop.step", cfg["loop"]["times"], W)
     for i, layer in enumerate(cfg["layers"]):
         p, mx = f"l{i}.", layer["mixer"]
+        if sandwich:
+            H, m = mx["heads"], p + "mix."
+            G = mx.get("kv_heads", H)
+            for k in ("norm1", "norm1b") + (("norm2", "norm2b") if layer["mlp"] else ()):
+                ones(p + k, W)
+            for k, n in (("q", H * mx["dim"]), ("k", G * mx["dim"]), ("v", G * mx["vdim"])):
+                mat(m + k, n, W)
+            mat(m + "o", W, H * mx["vdim"])
+            if layer["type"] == "gla":
+                r = cfg.get("gla_rank", 16)
+                mat(m + "g", H * mx["vdim"], W)
+                mat(m + "a1", r, W)
+                mat(m + "a2", H * mx["dim"], r)
+                zeros(m + "a2.b", H * mx["dim"])
+                ones(m + "norm", mx["vdim"])
+            else:
+                mat(m + "g", H, W)
+                for k, n in (("q", H * mx["dim"]), ("k", G * mx["dim"]), ("v", G * mx["vdim"]), ("o", W)):
+                    zeros(m + k + ".b", n)
+                ones(m + "q.norm", mx["dim"])
+                ones(m + "k.norm", mx["dim"])
+                mat(m + "rel", 32, H)
+                zeros(m + "pb", H)
+            mlp = layer["mlp"]
+            if mlp is not None and mlp["kind"] == "moe":
+                f = mlp["expert"]["ff"]
+                for e in range(mlp["router"]["experts"]):
+                    mat(f"{p}mlp.e{e}.up", f, W)
+                    mat(f"{p}mlp.e{e}.down", W, f)
+                mat(p + "mlp.router", mlp["router"]["experts"], W)
+                zeros(p + "mlp.router.b", mlp["router"]["experts"])
+            elif mlp is not None:
+                mat(p + "mlp.up", mlp["ff"], W)
+                mat(p + "mlp.down", W, mlp["ff"])
+                zeros(p + "mlp.act", 2)
+            continue
         ones(p + "norm1")
         if layer["type"] == "latent_attention":
             H, r = mx["heads"], mx["kv_rank"]
@@ -163,13 +226,13 @@ def token_lm_state_dict(cfg: dict, seed: int = 0, device="cpu") -> dict[str, Ten
             for k in ("z", "x", "g"):
                 mat(p + "mix." + k, n, W)
             for k in ("z.b", "x.b"):
-                sd[p + "mix." + k] = torch.zeros(n, dtype=torch.bfloat16, device=device)
+                zeros(p + "mix." + k, n)
             mat(p + "mix.o", W, n)
         if layer["mlp"] is not None:
             f = layer["mlp"]["ff"]
             mat(p + "mlp.gate", f, W)
             mat(p + "mlp.up", f, W)
             mat(p + "mlp.down", W, f)
-    ones("final.norm")
+    ones("final.norm", *((W,) if sandwich else ()))
     mat("head", cfg["vocab"], W)
     return sd
