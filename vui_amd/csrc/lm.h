@@ -93,7 +93,8 @@ struct LmGemm {
   float act_pos, act_neg;
   // entries (row top + choice) sorted by expert, every expert's padded with -1 to whole tiles; expert of each tile
   const int32_t *ent, *tile_e, *n_tiles;
-  int top, max_tiles;
+  int top, max_tiles, tile_rows;
+  int sorted;      // X holds a row per entry instead of a row per position
 };
 int launch_lm_gemm(int dtype, int epi, const LmGemm& g, int nz, hipStream_t st);
 int launch_lm_embed(int dtype, const int64_t* tokens, const void* table, float* x, void* xt, float* ssq, int rows, int width,
@@ -169,8 +170,14 @@ struct RowArgs {
   void* xt;                // (rows, w64) tiled
   void* xcat;              // (rows, 2 w64) tiled: [x | embedding]
   int to_cat;
+  // router logits of the normed row (few rows), or rlog nullptr
+  const void* w_router;
+  const float* router_bias;
+  int experts16;
+  float* rlog;             // (M, experts16)
 };
 int launch_lm_rows(const RowArgs& a, hipStream_t st);
+bool lm_rows_routes(int M, int experts16);  // it takes the router's product too
 
 // ---- attention with sigmoid weights (sigattn.hip) ----
 struct SigAttnArgs {
@@ -196,6 +203,7 @@ int launch_sig_prep(const SigAttnArgs& a, hipStream_t st);    // norms, temperat
 int launch_sig_pieces(const SigAttnArgs& a, hipStream_t st);  // few rows: pieces, merge, gate
 int launch_sig_prompt(const SigAttnArgs& a, hipStream_t st);  // block of one sequence, bf16
 bool sig_mfma_ok(const vui_lm_dims& d);
+bool sig_step_fused(int dtype, const LmRows& rows, const vui_lm_dims& d);  // launch_sig_pieces norms and appends by itself
 int sig_splits(int M, int heads, int kv_heads);
 
 // ---- gated linear attention (gla.hip) ----
@@ -225,6 +233,13 @@ struct RouteArgs {
   int32_t *ent, *tile_e, *n_tiles;
 };
 int launch_moe_route(const RouteArgs& a, hipStream_t st);
+// rows of a tiled operand (rows, cols) copied to their entries' places
+int launch_moe_gather(int dtype, const RouteArgs& a, const void* x, void* out, int cols, int max_tiles, hipStream_t st);
+// rows of the tiles an expert's entries are padded to
+static inline int moe_tile_rows(int dtype, int M, int entries, int experts) {
+  if (M <= 16) return 16;
+  return dtype == VUI_DTYPE_BF16 && entries / experts >= 64 ? 64 : 32;
+}
 static inline int moe_max_tiles(int entries, int experts, int tile_rows) {
   const int a = entries / tile_rows + experts;
   return entries < a ? entries : a;
@@ -246,7 +261,7 @@ struct vui_lm_ctx {
   float* layers_out;
   int expand_from;
   // sandwich layers
-  void *xcat, *raw, *ffa;
+  void *xcat, *raw, *ffa, *xg;
   float *y, *bsum, *gupd, *gdec, *rlog, *share;
   int32_t *choice, *ent, *tile_e, *n_tiles;
   int attn_from, gla_from;

@@ -50,11 +50,12 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
   const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63;
   const int l16 = lane & 15, kg = lane >> 4;
   const int MT = MOE ? p.max_tiles : (p.M + 16 * MB - 1) / (16 * MB);
-  const int m0 = ((int)blockIdx.x % MT) * 16 * MB, nb0 = ((int)blockIdx.x / MT) * NB;
+  // tiles of an expert that share features run on one XCD, whose cache then holds those weights: workgroup i is on XCD i % 8
+  const int slice = MOE ? (int)blockIdx.x >> 3 : (int)blockIdx.x, t = slice % MT;
+  const int m0 = t * 16 * MB, nb0 = (MOE ? (slice / MT) * 8 + ((int)blockIdx.x & 7) : slice / MT) * NB;
   size_t wz = blockIdx.z * p.wz;
   if (MOE) {
-    const int t = (int)blockIdx.x % MT;
-    if (t >= p.n_tiles[0]) return;  // uniform
+    if (t >= p.n_tiles[0] || nb0 >= (p.N >> 4)) return;  // uniform
     wz = (size_t)p.tile_e[t] * p.wz;
   }
   const int nsteps = p.K >> 6;
@@ -65,10 +66,10 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
   const T* wr[NB];
 #pragma unroll
   for (int j = 0; j < MB; ++j) {
-    if (EPI == LM_MOE_UP) {
+    if (EPI == LM_MOE_UP && !p.sorted) {
       const int e = p.ent[m0 + 16 * j + l16], r = min(max(e, 0) / p.top, p.x_rows - 1);
       xr[j] = (const T*)p.X + (size_t)(r >> 4) * nsteps * 1024 + ((r & 15) + 16 * kg) * EP;
-    } else if (EPI == LM_MOE_DOWN) {
+    } else if (MOE) {
       xr[j] = (const T*)p.X + (size_t)((m0 >> 4) + j) * nsteps * 1024 + lane * EP;
     } else if (LOGITS && p.rowmap) {
       const int r = min(max(p.rowmap[min(m0 + 16 * j + l16, p.M - 1)], 0), p.x_rows - 1);
@@ -315,7 +316,8 @@ __global__ __launch_bounds__(64 * WAVES) void lm_gemm_kernel(const LmGemm p) {
 template <typename T, int MB, int NB, int WAVES, int EPI>
 static int go(const LmGemm& g, int nz, hipStream_t st) {
   const bool moe = EPI == LM_MOE_UP || EPI == LM_MOE_DOWN;
-  const int tiles = (moe ? g.max_tiles : (g.M + 16 * MB - 1) / (16 * MB)) * ((g.N / 16 + NB - 1) / NB);
+  const int nt = (g.N / 16 + NB - 1) / NB;
+  const int tiles = moe ? g.max_tiles * ((nt + 7) & ~7) : (g.M + 16 * MB - 1) / (16 * MB) * nt;
   hipLaunchKernelGGL((lm_gemm_kernel<T, MB, NB, WAVES, EPI>), dim3((unsigned)tiles, 1, nz), dim3(64 * WAVES), 0, st, g);
   HIP_TRY(hipGetLastError());
   return VUI_OK;
@@ -325,6 +327,18 @@ static int go(const LmGemm& g, int nz, hipStream_t st) {
 template <typename T>
 static int pick(int epi, const LmGemm& g, int nz, hipStream_t st) {
   const bool few = g.M <= 16;
+  // many rows: tiles of 64 x 64, or 64 x 32 where the former would leave half of the chip idle
+  const long tiles = (long)((g.M + 63) / 64) * ((g.N + 63) / 64);
+  if (sizeof(T) == 2 && g.M >= 256 && tiles >= 64) {
+    const bool wide = tiles >= 160;
+    if (epi == LM_PROJ) return wide ? go<T, 4, 4, 4, LM_PROJ>(g, nz, st) : go<T, 4, 2, 4, LM_PROJ>(g, nz, st);
+    if (epi == LM_PLAIN) return wide ? go<T, 4, 4, 4, LM_PLAIN>(g, nz, st) : go<T, 4, 2, 4, LM_PLAIN>(g, nz, st);
+    if (epi == LM_ACT) return wide ? go<T, 4, 4, 4, LM_ACT>(g, nz, st) : go<T, 4, 2, 4, LM_ACT>(g, nz, st);
+  }
+  if (sizeof(T) == 2 && g.tile_rows == 64) {
+    if (epi == LM_MOE_UP) return go<T, 4, 4, 4, LM_MOE_UP>(g, nz, st);
+    if (epi == LM_MOE_DOWN) return go<T, 4, 4, 4, LM_MOE_DOWN>(g, nz, st);
+  }
   switch (epi) {
     case LM_IN_ATTN: return few ? go<T, 1, 2, 8, LM_IN_ATTN>(g, nz, st) : go<T, 2, 2, 4, LM_IN_ATTN>(g, nz, st);
     case LM_IN_GRU_STEP: return go<T, 1, 3, 8, LM_IN_GRU_STEP>(g, nz, st);

@@ -2,6 +2,7 @@
 // the (row, choice) entries sorted by expert, every expert's padded to whole tiles of the products that follow.
 #include "common.h"
 #include "lm.h"
+#include "tile.h"
 
 // one wave; picks in order of falling logits, so "behind the last pick" needs no list of what was taken
 __device__ __forceinline__ void route_row(const RouteArgs& p, int m) {
@@ -86,6 +87,28 @@ int launch_moe_route(const RouteArgs& a, hipStream_t st) {
     hipLaunchKernelGGL(moe_top_kernel, dim3((a.M + 3) / 4), dim3(256), 0, st, a);
     hipLaunchKernelGGL(moe_sort_kernel<false>, dim3(1), dim3(1024), 0, st, a);
   }
+  HIP_TRY(hipGetLastError());
+  return VUI_OK;
+}
+
+// one workgroup per 16 entries and slice of the columns; a thread copies pieces of 16 bytes
+template <typename T>
+__global__ __launch_bounds__(256) void moe_gather_kernel(const RouteArgs p, const T* x, T* out, int nk) {
+  constexpr int EP = Tl<T>::EP, P = 16 / EP;
+  const int b = blockIdx.x, tid = threadIdx.x, lane = tid & 63;
+  if (b * 16 >= p.n_tiles[0] * p.tile_rows) return;
+  const int r = min(max(p.ent[b * 16 + (lane & 15)], 0) / p.top, p.M - 1);  // padding entries read row 0
+  const T* src = x + (size_t)(r >> 4) * nk * 1024 + ((r & 15) + 16 * (lane >> 4)) * EP;
+  T* dst = out + (size_t)b * nk * 1024 + lane * EP;
+  for (int i = blockIdx.y * 4 + (tid >> 6); i < nk * P; i += 4 * gridDim.y)
+    *reinterpret_cast<uint4*>(dst + (size_t)i * 64 * EP) = *reinterpret_cast<const uint4*>(src + (size_t)i * 64 * EP);
+}
+
+int launch_moe_gather(int dtype, const RouteArgs& a, const void* x, void* out, int cols, int max_tiles, hipStream_t st) {
+  if (cols < 64 || (cols & 63) || max_tiles < 1 || (a.tile_rows & 15)) { vui_set_error("expert gather: bad shape"); return VUI_EINVAL; }
+  const dim3 grid(max_tiles * (a.tile_rows / 16), 2);
+  if (dtype == VUI_DTYPE_F32) hipLaunchKernelGGL(moe_gather_kernel<float>, grid, dim3(256), 0, st, a, (const float*)x, (float*)out, cols >> 6);
+  else hipLaunchKernelGGL(moe_gather_kernel<bf16_t>, grid, dim3(256), 0, st, a, (const bf16_t*)x, (bf16_t*)out, cols >> 6);
   HIP_TRY(hipGetLastError());
   return VUI_OK;
 }

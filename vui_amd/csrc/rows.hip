@@ -1,97 +1,167 @@
 // Residual rows of sandwich layers: what a sublayer produced is normed and added, and the next sublayer's input is
 // normed, in one pass over the row.  fp32 throughout; a norm divides each of `groups` equal parts of the row by its own
-// root mean square.  One workgroup per row, the row in LDS.
+// root mean square.  One workgroup per row, the row in LDS; few rows take workgroups of 1024 threads, because a row is a
+// chain of dependent trips.  For few rows the router of an expert layer reads the normed row here as well.
 #include "common.h"
 #include "lm.h"
 #include "tile.h"
 
-#define ROWS_THREADS 256
-
-// root mean squares of the parts of `v` (width floats in LDS) -> 1 / rms in inv[g]; every wave takes parts in turn
-__device__ __forceinline__ void part_scales(const float* v, float* inv, int width, int groups, float eps) {
+// root mean squares of the parts of `v` (width floats in LDS) -> 1 / rms in inv[g].  A team of waves sums a part when
+// there are fewer parts than waves; red: max(groups, waves) floats.
+template <int NT>
+__device__ __forceinline__ void part_scales(const float* v, float* inv, float* red, int width, int groups, float eps) {
+  constexpr int WAVES = NT / 64;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, n = width / groups;
-  if (groups >= ROWS_THREADS / 64) {
-    for (int g = wave; g < groups; g += ROWS_THREADS / 64) {
-      float s = 0.f;
-      for (int i = lane; i < n; i += 64) { const float a = v[g * n + i]; s = fmaf(a, a, s); }
-      s = wave_sum(s);
-      if (lane == 0) inv[g] = 1.0f / sqrtf(s / (float)n + eps);
-    }
-    __syncthreads();
-    return;
-  }
-  // few parts: all waves share each
-  __shared__ float red[4][ROWS_THREADS / 64];
-  for (int g = 0; g < groups; ++g) {
+  const int wp = groups < WAVES ? WAVES / groups : 1, teams = WAVES / wp, sub = wave % wp;
+  for (int g = wave / wp; g < groups && wave < teams * wp; g += teams) {
+    const float* q = v + g * n;
     float s = 0.f;
-    for (int i = threadIdx.x; i < n; i += ROWS_THREADS) { const float a = v[g * n + i]; s = fmaf(a, a, s); }
+#pragma unroll 4
+    for (int i = sub * 64 + lane; i < n; i += wp * 64) s = fmaf(q[i], q[i], s);
     s = wave_sum(s);
-    if (lane == 0) red[g][wave] = s;
+    if (lane == 0) red[g * wp + sub] = s;
   }
   __syncthreads();
-  if ((int)threadIdx.x < groups) {
-    const float* r = red[threadIdx.x];
-    inv[threadIdx.x] = 1.0f / sqrtf(((r[0] + r[1]) + (r[2] + r[3])) / (float)n + eps);
+  for (int g = threadIdx.x; g < groups; g += NT) {
+    float s = 0.f;
+    for (int w = 0; w < wp; ++w) s += red[g * wp + w];
+    inv[g] = 1.0f / sqrtf(s / (float)n + eps);
   }
   __syncthreads();
 }
 
-template <typename T>
-__global__ __launch_bounds__(ROWS_THREADS) void lm_rows_kernel(const RowArgs p) {
-  extern __shared__ __align__(16) float rl[];  // row (w64), 1 / rms (groups)
-  float* inv = rl + p.w64;
+// router logits of the normed row in LDS: a wave takes blocks of 64 columns, a lane 16 columns of one expert
+template <typename T, int NT>
+__device__ __forceinline__ void route_logits(const RowArgs& p, const float* v, float* red, int m) {
+  constexpr int WAVES = NT / 64, EP = Tl<T>::EP, P = 16 / EP;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, l16 = lane & 15, kg = lane >> 4, nk = p.w64 >> 6;
+  for (int b = 0; b < p.experts16 >> 4; ++b) {
+    const T* w = (const T*)p.w_router + (size_t)b * nk * 1024 + lane * EP;
+    float s = 0.f;
+    for (int k = wave; k < nk; k += WAVES) {
+      uint4 q[P];
+#pragma unroll
+      for (int h = 0; h < P; ++h) q[h] = *reinterpret_cast<const uint4*>(w + (size_t)k * 1024 + 64 * EP * h);
+      const float* c = v + k * 64 + kg * 16;
+#pragma unroll
+      for (int h = 0; h < P; ++h) {
+        const T* e = reinterpret_cast<const T*>(&q[h]);
+#pragma unroll
+        for (int i = 0; i < EP; ++i) s = fmaf(El<T>::ld(e + i), c[h * EP + i], s);
+      }
+    }
+    s = rows_sum(s);
+    if (kg == 0) red[wave * p.experts16 + b * 16 + l16] = s;
+  }
+  __syncthreads();
+  for (int e = threadIdx.x; e < p.experts16; e += NT) {
+    float s = p.router_bias[e];
+    for (int w = 0; w < WAVES; ++w) s += red[w * p.experts16 + e];
+    p.rlog[(size_t)m * p.experts16 + e] = s;
+  }
+}
+
+template <typename T, int NT>
+__global__ __launch_bounds__(NT) void lm_rows_kernel(const RowArgs p) {
+  extern __shared__ __align__(16) float rl[];  // row (w64), 1 / rms (groups), sums
+  float *inv = rl + p.w64, *red = inv + p.groups;
   const int m = blockIdx.x, tid = threadIdx.x, n = p.width / p.groups;
   float* xr = p.x + (size_t)m * p.w64;
-  const size_t row16 = (size_t)m;
+  const bool add = !p.tokens && !p.step;
   if (p.tokens) {
     int64_t t = p.tokens[m];
     t = t < 0 ? 0 : (t >= p.vocab ? p.vocab - 1 : t);
-    for (int k = tid; k < p.w64; k += ROWS_THREADS) {
+    for (int k = tid; k < p.w64; k += NT) {
       const float v = k < p.width ? El<T>::ld((const T*)p.embed + (size_t)t * p.width + k) * p.emb_scale : 0.f;
       rl[k] = v;
-      if (p.xcat) El<T>::st((T*)p.xcat + tl_off<T>((int)row16, p.w64 + k, 2 * p.w64), v);
+      if (p.xcat) El<T>::st((T*)p.xcat + tl_off<T>(m, p.w64 + k, 2 * p.w64), v);
     }
     __syncthreads();
-  } else if (p.step) {
-    for (int k = tid; k < p.w64; k += ROWS_THREADS) rl[k] = k < p.width ? p.y[(size_t)m * p.ldy + k] + p.step[k] : 0.f;
-    __syncthreads();
-  } else {
-    for (int k = tid; k < p.w64; k += ROWS_THREADS) {
-      float v = 0.f;
-      if (k < p.width) {
-        if (p.share) {
-          for (int c = 0; c < p.top; ++c) v = fmaf(p.share[(size_t)m * p.top + c], p.y[((size_t)m * p.top + c) * p.ldy + k], v);
+  }
+  float4 old = make_float4(0.f, 0.f, 0.f, 0.f), post = old, next = old;  // of the thread's first quad, requested ahead of use
+  const int k1 = min(tid * 4, p.w64 - 4);
+  if (add) {
+    old = *reinterpret_cast<const float4*>(xr + k1);
+    post = *reinterpret_cast<const float4*>(p.post + k1);
+  }
+  if (p.next) next = *reinterpret_cast<const float4*>(p.next + k1);
+  if (!p.tokens) {
+    for (int k = tid * 4; k < p.w64; k += NT * 4) {
+      tl_f32x4 v = {0.f, 0.f, 0.f, 0.f};
+      if (k < p.ldy) {  // what is behind the width is zero
+        if (add && p.share) {
+          const float *y = p.y + (size_t)m * p.top * p.ldy + k, *s = p.share + (size_t)m * p.top;
+#pragma unroll 4
+          for (int c = 0; c < p.top; ++c) v += s[c] * *reinterpret_cast<const tl_f32x4*>(y + (size_t)c * p.ldy);
         } else {
-          v = p.y[(size_t)m * p.ldy + k];
+          v = *reinterpret_cast<const tl_f32x4*>(p.y + (size_t)m * p.ldy + k);
         }
       }
-      rl[k] = v;
+      if (p.step) v += *reinterpret_cast<const tl_f32x4*>(p.step + k);
+      *reinterpret_cast<tl_f32x4*>(rl + k) = v;
     }
     __syncthreads();
-    part_scales(rl, inv, p.width, p.groups, p.eps);
-    for (int k = tid; k < p.width; k += ROWS_THREADS) rl[k] = xr[k] + rl[k] * inv[k / n] * p.post[k];
-    __syncthreads();
   }
-  for (int k = tid; k < p.w64; k += ROWS_THREADS) {
-    xr[k] = rl[k];
-    if (p.layer_out && k < p.width) p.layer_out[(size_t)m * p.width + k] = rl[k];
-    if (p.to_cat) El<T>::st((T*)p.xcat + tl_off<T>((int)row16, k, 2 * p.w64), rl[k]);
+  if (add) part_scales<NT>(rl, inv, red, p.width, p.groups, p.eps);
+  for (int k = tid * 4; k < p.w64; k += NT * 4) {
+    tl_f32x4 v = *reinterpret_cast<const tl_f32x4*>(rl + k);
+    if (add) {
+      if (k != k1) {
+        old = *reinterpret_cast<const float4*>(xr + k);
+        post = *reinterpret_cast<const float4*>(p.post + k);
+      }
+      const float o[4] = {old.x, old.y, old.z, old.w}, w[4] = {post.x, post.y, post.z, post.w};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = k + i < p.width ? o[i] + v[i] * inv[(k + i) / n] * w[i] : 0.f;
+      *reinterpret_cast<tl_f32x4*>(rl + k) = v;
+    }
+    *reinterpret_cast<tl_f32x4*>(xr + k) = v;
+    const float f[4] = {v[0], v[1], v[2], v[3]};
+    if (p.to_cat) Tl<T>::st4((T*)p.xcat + tl_off<T>(m, k, 2 * p.w64), f);
+    if (p.layer_out)
+      for (int i = 0; i < 4; ++i) if (k + i < p.width) p.layer_out[(size_t)m * p.width + k + i] = f[i];
   }
   if (!p.next) return;
-  part_scales(rl, inv, p.width, p.groups, p.eps);
-  for (int k = tid; k < p.w64; k += ROWS_THREADS)
-    El<T>::st((T*)p.xt + tl_off<T>((int)row16, k, p.w64), k < p.width ? rl[k] * inv[k / n] * p.next[k] : 0.f);
+  __syncthreads();
+  part_scales<NT>(rl, inv, red, p.width, p.groups, p.eps);
+  for (int k = tid * 4; k < p.w64; k += NT * 4) {
+    if (k != k1) next = *reinterpret_cast<const float4*>(p.next + k);
+    const float w[4] = {next.x, next.y, next.z, next.w};
+    float f[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) f[i] = k + i < p.width ? rl[k + i] * inv[(k + i) / n] * w[i] : 0.f;
+    T* dst = (T*)p.xt + tl_off<T>(m, k, p.w64);
+    Tl<T>::st4(dst, f);
+    if (p.rlog) {  // the router reads what the product of more rows would: the rounded row
+      T r[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) { El<T>::st(&r[i], f[i]); f[i] = El<T>::ld(&r[i]); }
+      *reinterpret_cast<float4*>(rl + k) = make_float4(f[0], f[1], f[2], f[3]);
+    }
+  }
+  if (!p.rlog) return;
+  __syncthreads();
+  route_logits<T, NT>(p, rl, red, m);
+}
+
+bool lm_rows_routes(int M, int experts16) { return M <= 16 && experts16 <= 128; }
+
+template <typename T, int NT>
+static int rows_go(const RowArgs& a, hipStream_t st) {
+  const int teams = a.groups < NT / 64 ? NT / 64 : a.groups, sums = a.rlog ? NT / 64 * a.experts16 : 0;
+  const size_t lds = ((size_t)a.w64 + a.groups + (sums > teams ? sums : teams)) * 4;
+  if (lds > 128 * 1024) { vui_set_error("lm rows: width %d too large", a.width); return VUI_EINVAL; }
+  if (lds > 60 * 1024) HIP_TRY(hipFuncSetAttribute((const void*)lm_rows_kernel<T, NT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+  hipLaunchKernelGGL((lm_rows_kernel<T, NT>), dim3(a.M), dim3(NT), lds, st, a);
+  HIP_TRY(hipGetLastError());
+  return VUI_OK;
 }
 
 int launch_lm_rows(const RowArgs& a, hipStream_t st) {
-  if (a.M < 1 || a.groups < 1 || a.width % a.groups || a.w64 < a.width || (a.w64 & 63)) { vui_set_error("lm rows: bad shape M=%d width=%d groups=%d", a.M, a.width, a.groups); return VUI_EINVAL; }
-  const size_t lds = ((size_t)a.w64 + a.groups) * 4;
-  if (lds > 128 * 1024) { vui_set_error("lm rows: width %d too large", a.width); return VUI_EINVAL; }
-  const bool f32 = a.dtype == VUI_DTYPE_F32;
-  if (lds > 60 * 1024)
-    HIP_TRY(hipFuncSetAttribute(f32 ? (const void*)lm_rows_kernel<float> : (const void*)lm_rows_kernel<bf16_t>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-  if (f32) hipLaunchKernelGGL(lm_rows_kernel<float>, dim3(a.M), dim3(ROWS_THREADS), lds, st, a);
-  else hipLaunchKernelGGL(lm_rows_kernel<bf16_t>, dim3(a.M), dim3(ROWS_THREADS), lds, st, a);
-  HIP_TRY(hipGetLastError());
-  return VUI_OK;
+  if (a.M < 1 || a.groups < 1 || a.width % a.groups || a.w64 < a.width || (a.w64 & 63) || (a.ldy & 3) || (a.rlog && !lm_rows_routes(a.M, a.experts16))) {
+    vui_set_error("lm rows: bad shape M=%d width=%d groups=%d", a.M, a.width, a.groups);
+    return VUI_EINVAL;
+  }
+  if (a.M <= 64) return a.dtype == VUI_DTYPE_F32 ? rows_go<float, 1024>(a, st) : rows_go<bf16_t, 1024>(a, st);
+  return a.dtype == VUI_DTYPE_F32 ? rows_go<float, 256>(a, st) : rows_go<bf16_t, 256>(a, st);
 }

@@ -1,8 +1,9 @@
 // Sandwich layers of the token language models: x <- x + norm(mixer(norm(x))), then x <- x + norm(ff(norm(x))).  See
 // include/vui_lm.h and lm.hip, which holds the context and the C ABI.
 //
-// Launches: input projection, mixer (sigmoid attention 3, or 2 for a block of a prompt; gated linear attention 1, by
-// chunks 3), output projection, rows, up, down, rows; an expert layer adds the router's product and 1-2 for routing.
+// Launches: input projection, mixer (sigmoid attention 2, portions of a prompt 3, blocks of one 2; gated linear
+// attention 1, by chunks 3), output projection, rows, up, down, rows; an expert layer adds 1 for routing, with more rows than
+// 16 the router's product, 2 for routing and 1 that puts the rows in order.
 // The rows launch (rows.hip) norms and adds what a sublayer produced and norms what the next one reads.
 #include <string.h>
 
@@ -53,7 +54,7 @@ bool sandwich_pointers_ok(const vui_lm_config& c, const vui_lm_layer& L) {
 size_t sandwich_carve(const vui_lm_config* c, const vui_lm_layer* layers, vui_lm_ctx* x, char* base) {
   const size_t e = lm_esz(*c);
   const size_t R = lm_pad(c->max_rows < 16 ? 16 : c->max_rows, 16);
-  size_t q = 0, raw = 0, ac = 0, pt = 0, ff = 0, yr = R, bs = 0, up = 0, de = 0, rl = 0, ch = 0, en = 0, ti = 0;
+  size_t q = 0, raw = 0, ac = 0, pt = 0, ff = 0, yr = R, bs = 0, up = 0, de = 0, rl = 0, ch = 0, en = 0, ti = 0, xg = 0;
   bool loops = false;
   vui_lm_dims d;
   memset(&d, 0, sizeof(d));
@@ -74,9 +75,13 @@ size_t sandwich_carve(const vui_lm_config* c, const vui_lm_layer* layers, vui_lm
       mx(pt, rows * H * d.vdim16);
     }
     if (L.experts > 0) {
-      const size_t n = R * L.top, t16 = moe_max_tiles(n, L.experts, 16), t32 = moe_max_tiles(n, L.experts, 32);
-      const size_t rows = t16 * 16 > t32 * 32 ? t16 * 16 : t32 * 32;
-      mx(ff, rows * d.ff64); mx(en, rows); mx(ti, t16); mx(yr, n); mx(ch, n); mx(rl, R * d.experts16);
+      const size_t n = R * L.top;
+      for (int tr = 16; tr <= 64; tr *= 2) {
+        const size_t tiles = moe_max_tiles(n, L.experts, tr), rows = tiles * tr;
+        mx(ff, rows * d.ff64); mx(en, rows); mx(ti, tiles);
+        if (tr > 16) mx(xg, rows * d.w64);
+      }
+      mx(yr, n); mx(ch, n); mx(rl, R * d.experts16);
     } else {
       mx(ff, R * d.ff64);
     }
@@ -93,6 +98,7 @@ size_t sandwich_carve(const vui_lm_config* c, const vui_lm_layer* layers, vui_lm
   TAKE(act, void*, ac * e);
   TAKE(y, float*, yr * d.w16 * 4);
   TAKE(ffa, void*, ff * e);
+  TAKE(xg, void*, xg * e);
   TAKE(bsum, float*, bs * 4);
   TAKE(gupd, float*, up * 4);
   TAKE(gdec, float*, de * 4);
@@ -143,7 +149,7 @@ static int mixer(vui_lm_ctx* x, int l, int M, const LmRows& rows, hipStream_t st
     a.q_norm = L.q_norm; a.k_norm = L.k_norm; a.temp_coef = L.temp_coef; a.temp_every = L.temp_every < 1 ? 1 : L.temp_every;
     a.bias = L.dist_bias; a.bias_len = L.bias_len; a.k_cache = L.k_cache; a.v_cache = L.v_cache;
     a.q = x->qu; a.q_z = (size_t)x->R16 * d.dim64; a.part = x->part; a.act = x->act;
-    if ((rc = launch_sig_prep(a, st))) return rc;
+    if (!sig_step_fused(x->c.dtype, rows, d) && (rc = launch_sig_prep(a, st))) return rc;
     if (rows.seq && M >= x->attn_from && x->c.dtype == VUI_DTYPE_BF16 && sig_mfma_ok(d)) {
       rc = launch_sig_prompt(a, st);
     } else {
@@ -166,18 +172,23 @@ static int feed_forward(vui_lm_ctx* x, int l, int M, const LmRows& rows, hipStre
     if ((rc = launch_lm_gemm(x->c.dtype, LM_ACT, up, 1, st))) return rc;
     return plain(x, d, rows, x->ffa, L.w_down, nullptr, M, d.out_rows, d.ff64, x->y, st);
   }
-  if ((rc = plain(x, d, rows, x->xt, L.w_router, L.router_bias, M, d.experts16, d.w64, x->rlog, st))) return rc;
+  if (!lm_rows_routes(M, d.experts16) && (rc = plain(x, d, rows, x->xt, L.w_router, L.router_bias, M, d.experts16, d.w64, x->rlog, st))) return rc;
   RouteArgs r;
   memset(&r, 0, sizeof(r));
-  r.M = M; r.E = L.experts; r.ldl = d.experts16; r.top = L.top; r.tile_rows = M <= 16 ? 16 : 32;
+  r.M = M; r.E = L.experts; r.ldl = d.experts16; r.top = L.top; r.tile_rows = moe_tile_rows(x->c.dtype, M, M * L.top, L.experts);
   r.logits = x->rlog; r.choice = x->choice; r.share = x->share; r.ent = x->ent; r.tile_e = x->tile_e; r.n_tiles = x->n_tiles;
   if ((rc = launch_moe_route(r, st))) return rc;
   up.ent = x->ent; up.tile_e = x->tile_e; up.n_tiles = x->n_tiles; up.top = L.top; up.wz = (size_t)d.ff16 * d.w64;
+  up.tile_rows = r.tile_rows;
   up.max_tiles = moe_max_tiles(M * L.top, L.experts, r.tile_rows);
+  if (M > 16) {
+    if ((rc = launch_moe_gather(x->c.dtype, r, x->xt, x->xg, d.w64, up.max_tiles, st))) return rc;
+    up.X = x->xg; up.sorted = 1;
+  }
   if ((rc = launch_lm_gemm(x->c.dtype, LM_MOE_UP, up, 1, st))) return rc;
   LmGemm down = product(x, d, rows, x->ffa, L.w_down, M, d.out_rows, d.ff64);
   down.ent = x->ent; down.tile_e = x->tile_e; down.n_tiles = x->n_tiles; down.top = L.top; down.wz = (size_t)d.out_rows * d.ff64;
-  down.max_tiles = up.max_tiles; down.out = x->y; down.ldo = d.out_rows;
+  down.max_tiles = up.max_tiles; down.tile_rows = r.tile_rows; down.out = x->y; down.ldo = d.out_rows;
   return launch_lm_gemm(x->c.dtype, LM_MOE_DOWN, down, 1, st);
 }
 
@@ -214,7 +225,11 @@ int sandwich_layers(vui_lm_ctx* x, const int64_t* tokens, int M, const LmRows& r
     r.share = nullptr; r.post = L.norm1b; r.layer_out = nullptr;
     if (L.ff > 0) {
       r.next = L.norm2; r.to_cat = 0;
-      if ((rc = launch_lm_rows(r, st))) return rc;
+      RowArgs mid = r;
+      if (L.experts > 0 && lm_rows_routes(M, d.experts16)) {
+        mid.w_router = L.w_router; mid.router_bias = L.router_bias; mid.experts16 = d.experts16; mid.rlog = x->rlog;
+      }
+      if ((rc = launch_lm_rows(mid, st))) return rc;
       if ((rc = feed_forward(x, l, M, rows, st))) return rc;
       r.post = L.norm2b;
       if (L.experts > 0) { r.share = x->share; r.top = L.top; }

@@ -2,6 +2,8 @@
 // simply add up.  Queries and keys are normed per head, a query is scaled by a temperature that grows with its
 // position, and a score gets a bias from a table over the distance.
 //
+// A decode step norms and appends inside the kernel of the pieces; portions of a prompt do it in a launch of their own.
+//
 // Caches: keys as tiled rows (tile.h), so that 16 keys x 64 columns are an operand of the matrix cores as they lie;
 // values in blocks of 16 dims x 32 positions, an operand of the second product.
 #include "common.h"
@@ -150,8 +152,46 @@ struct SigTile {
 // sigmoid of a score given t = -log2(e) score
 __device__ __forceinline__ float sig_weight(float t) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(t)); }
 
+// a normed row as a lane's part of an operand: columns 64 b + 16 kg .. + 15 in f[2 b], f[2 b + 1]; src: dim16 values
+template <int DB>
+__device__ __forceinline__ void sig_normed(const bf16_t* src, const float* w, int dim16, int dim, float eps, float mul, int kg, uint4* f) {
+  float v[DB][16], ss = 0.f;
+#pragma unroll
+  for (int b = 0; b < DB; ++b) {
+    const int col = b * 64 + kg * 16;
+    const bool live = col < dim16;
+    const uint4* q = reinterpret_cast<const uint4*>(src + (live ? col : 0));
+    const uint4 x[2] = {q[0], q[1]};
+#pragma unroll
+    for (int h = 0; h < 2; ++h) {
+      const uint32_t u[4] = {x[h].x, x[h].y, x[h].z, x[h].w};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        v[b][8 * h + 2 * i] = live ? bf_lo(u[i]) : 0.f;
+        v[b][8 * h + 2 * i + 1] = live ? bf_hi(u[i]) : 0.f;
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 16; ++i) ss = fmaf(v[b][i], v[b][i], ss);
+  }
+  const float r = mul / sqrtf(rows_sum(ss) / (float)dim + eps);
+#pragma unroll
+  for (int b = 0; b < DB; ++b) {
+    const int col = b * 64 + kg * 16;
+    const float* c = w + (col < dim16 ? col : 0);
+#pragma unroll
+    for (int i = 0; i < 16; ++i) v[b][i] *= r * c[i];
+#pragma unroll
+    for (int h = 0; h < 2; ++h)
+      f[2 * b + h] = make_uint4(f2bf2(v[b][8 * h], v[b][8 * h + 1]), f2bf2(v[b][8 * h + 2], v[b][8 * h + 3]),
+                                f2bf2(v[b][8 * h + 4], v[b][8 * h + 5]), f2bf2(v[b][8 * h + 6], v[b][8 * h + 7]));
+  }
+}
+
 // ---- pieces on the matrix cores (bf16): one workgroup per (row, up to 16 heads of one group, piece) ----
-template <int DB, int VT>
+// STEP (one position per slot): queries are normed here, and the wave that comes to the new position's tile norms its key,
+// puts key and value into its operands and appends them (workgroups of further heads of the group write the same).
+template <int DB, int VT, bool STEP>
 __global__ __launch_bounds__(256) void sig_piece_mfma_kernel(const SigAttnArgs p) {
   __shared__ __align__(16) float s_acc[4][VT * 256];
   const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, l16 = lane & 15, kg = lane >> 4;
@@ -166,9 +206,14 @@ __global__ __launch_bounds__(256) void sig_piece_mfma_kernel(const SigAttnArgs p
   const bf16_t* vb = (const bf16_t*)p.v_cache + ((size_t)slot * p.kv_heads + g) * p.d.s64 * p.d.vdim16 + lane * 8;
   const float* bias = p.bias + (size_t)head * p.bias_len;
   uint4 qf[2 * DB];
+  const bf16_t* row = (const bf16_t*)p.raw + (size_t)m * p.ld;
+  if (STEP) {
+    sig_normed<DB>(row + head * p.d.dim16, p.q_norm, p.d.dim16, p.dim, p.eps, sig_temp(p, pos), kg, qf);
+  } else {
 #pragma unroll
-  for (int i = 0; i < 2 * DB; ++i)
-    qf[i] = *reinterpret_cast<const uint4*>((const bf16_t*)p.q + head * p.q_z + ((size_t)(m >> 4) * DB * 2 + i) * 512 + ((m & 15) + 16 * kg) * 8);
+    for (int i = 0; i < 2 * DB; ++i)
+      qf[i] = *reinterpret_cast<const uint4*>((const bf16_t*)p.q + head * p.q_z + ((size_t)(m >> 4) * DB * 2 + i) * 512 + ((m & 15) + 16 * kg) * 8);
+  }
   tl_f32x4 acc[VT];
 #pragma unroll
   for (int d = 0; d < VT; ++d) acc[d] = tl_f32x4{0.f, 0.f, 0.f, 0.f};
@@ -181,6 +226,32 @@ __global__ __launch_bounds__(256) void sig_piece_mfma_kernel(const SigAttnArgs p
     for (int e = 0; e < 8; ++e) {
       const int j = k0 + 16 * (e >> 2) + 4 * kg + (e & 3);
       b[e] = bias[min(max(len - 1 - j, 0), p.bias_len - 1)];
+    }
+    if (STEP && pos == len - 1 && (pos >> 5) == (k0 >> 5)) {  // uniform; a position outside the slot is not stored
+      const SigCols cols = sig_cols(p);
+      uint4 nk[2 * DB];
+      sig_normed<DB>(row + cols.k + g * p.d.dim16, p.k_norm, p.d.dim16, p.dim, p.eps, 1.f, kg, nk);
+      const bool mine = l16 == (pos & 15);
+      bf16_t* ko = const_cast<bf16_t*>(kb) + (size_t)(pos >> 4) * DB * 1024;
+#pragma unroll
+      for (int i = 0; i < 2 * DB; ++i) {
+        if (mine && !(pos & 16)) t.kf[0][i] = nk[i];
+        if (mine && (pos & 16)) t.kf[1][i] = nk[i];
+        if (mine) *reinterpret_cast<uint4*>(ko + i * 512) = nk[i];
+      }
+      const bool vmine = kg == ((pos & 15) >> 2);
+      const int w = 2 * ((pos & 31) >> 4) + ((pos & 3) >> 1), sh = 16 * (pos & 1), e = 4 * ((pos & 31) >> 4) + (pos & 3);
+      bf16_t* vo = const_cast<bf16_t*>(vb) + (size_t)(pos >> 5) * nvb * 512 + e;
+#pragma unroll
+      for (int d = 0; d < VT; ++d) {
+        const bf16_t nv = row[cols.v + g * p.d.vdim16 + min(d, nvb - 1) * 16 + l16];
+        const uint32_t keep = 0xffffu << (16 - sh), put = (uint32_t)nv << sh;
+        if (vmine && w == 0) t.vf[d].x = (t.vf[d].x & keep) | put;
+        if (vmine && w == 1) t.vf[d].y = (t.vf[d].y & keep) | put;
+        if (vmine && w == 2) t.vf[d].z = (t.vf[d].z & keep) | put;
+        if (vmine && w == 3) t.vf[d].w = (t.vf[d].w & keep) | put;
+        if (vmine && d < nvb) vo[(size_t)d * 512] = nv;
+      }
     }
     __builtin_amdgcn_sched_barrier(0);
     tl_f32x4 s[2];
@@ -310,6 +381,7 @@ __global__ __launch_bounds__(64 * SIGP_WAVES) void sig_prompt_kernel(const SigAt
 }
 
 // ---- launchers ----
+bool sig_step_fused(int dtype, const LmRows& rows, const vui_lm_dims& d) { return dtype == VUI_DTYPE_BF16 && !rows.seq && sig_mfma_ok(d); }
 bool sig_mfma_ok(const vui_lm_dims& d) { return d.dim64 <= 256 && d.vdim16 <= 256; }
 
 // pieces per row: as many workgroups as keep the chip busy
@@ -330,7 +402,9 @@ int launch_sig_prep(const SigAttnArgs& a, hipStream_t st) {
 template <int DB, int VT>
 static void piece_go(const SigAttnArgs& a, hipStream_t st) {
   const int per = a.heads / a.kv_heads;
-  hipLaunchKernelGGL((sig_piece_mfma_kernel<DB, VT>), dim3(a.M, a.kv_heads * ((per + 15) / 16), a.n_splits), dim3(256), 0, st, a);
+  const dim3 grid(a.M, a.kv_heads * ((per + 15) / 16), a.n_splits);
+  if (a.rows.seq) hipLaunchKernelGGL((sig_piece_mfma_kernel<DB, VT, false>), grid, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((sig_piece_mfma_kernel<DB, VT, true>), grid, dim3(256), 0, st, a);
 }
 template <int DB, int VT>
 static void prompt_go(const SigAttnArgs& a, hipStream_t st) {
