@@ -149,6 +149,15 @@ struct ScanArgs {
 int launch_gated_scan(const ScanArgs& a, hipStream_t st);
 #define LM_SCAN_CHUNK 32
 
+// ---- expert routing: logits to choices, shares and entries sorted by expert ----
+struct RouteArgs {
+  int M, E, ldl, top, tile_rows;
+  const float* logits;     // (M, ldl)
+  int32_t* choice;         // (M, top)
+  float* share;            // (M, top)
+  int32_t *ent, *tile_e, *n_tiles;
+};
+
 // ---- residual rows of sandwich layers (rows.hip) ----
 struct RowArgs {
   int dtype, M, width, w64, ldy, groups;
@@ -175,6 +184,7 @@ struct RowArgs {
   const float* router_bias;
   int experts16;
   float* rlog;             // (M, experts16)
+  RouteArgs route;         // of a single row: routed as well
 };
 int launch_lm_rows(const RowArgs& a, hipStream_t st);
 bool lm_rows_routes(int M, int experts16);  // it takes the router's product too
@@ -225,13 +235,6 @@ bool gla_chunk_ok(const vui_lm_dims& d);
 #define LM_GLA_CHUNK 32
 
 // ---- expert routing (moe.hip) ----
-struct RouteArgs {
-  int M, E, ldl, top, tile_rows;
-  const float* logits;     // (M, ldl)
-  int32_t* choice;         // (M, top)
-  float* share;            // (M, top)
-  int32_t *ent, *tile_e, *n_tiles;
-};
 int launch_moe_route(const RouteArgs& a, hipStream_t st);
 // rows of a tiled operand (rows, cols) copied to their entries' places
 int launch_moe_gather(int dtype, const RouteArgs& a, const void* x, void* out, int cols, int max_tiles, hipStream_t st);

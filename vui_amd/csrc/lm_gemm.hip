@@ -339,6 +339,13 @@ static int pick(int epi, const LmGemm& g, int nz, hipStream_t st) {
     if (epi == LM_MOE_UP) return go<T, 4, 4, 4, LM_MOE_UP>(g, nz, st);
     if (epi == LM_MOE_DOWN) return go<T, 4, 4, 4, LM_MOE_DOWN>(g, nz, st);
   }
+  // few rows and few features: one block of features per workgroup, so that more of the chip takes part
+  if (few && (long)g.N * (g.max_tiles > 0 ? g.max_tiles : 1) <= 4096) {
+    if (epi == LM_PROJ) return go<T, 1, 1, 16, LM_PROJ>(g, nz, st);
+    if (epi == LM_ACT) return go<T, 1, 1, 16, LM_ACT>(g, nz, st);
+    if (epi == LM_MOE_UP) return go<T, 1, 1, 16, LM_MOE_UP>(g, nz, st);
+    if (epi == LM_MOE_DOWN) return go<T, 1, 1, 16, LM_MOE_DOWN>(g, nz, st);
+  }
   switch (epi) {
     case LM_IN_ATTN: return few ? go<T, 1, 2, 8, LM_IN_ATTN>(g, nz, st) : go<T, 2, 2, 4, LM_IN_ATTN>(g, nz, st);
     case LM_IN_GRU_STEP: return go<T, 1, 3, 8, LM_IN_GRU_STEP>(g, nz, st);

@@ -2,8 +2,8 @@
 // include/vui_lm.h and lm.hip, which holds the context and the C ABI.
 //
 // Launches: input projection, mixer (sigmoid attention 2, portions of a prompt 3, blocks of one 2; gated linear
-// attention 1, by chunks 3), output projection, rows, up, down, rows; an expert layer adds 1 for routing, with more rows than
-// 16 the router's product, 2 for routing and 1 that puts the rows in order.
+// attention 1, by chunks 3), output projection, rows, up, down, rows; an expert layer adds 1 for routing (none for one row), with more
+// rows than 16 the router's product, 2 for routing and 1 that puts the rows in order.
 // The rows launch (rows.hip) norms and adds what a sublayer produced and norms what the next one reads.
 #include <string.h>
 
@@ -161,6 +161,15 @@ static int mixer(vui_lm_ctx* x, int l, int M, const LmRows& rows, hipStream_t st
   return plain(x, d, rows, x->act, L.w_out, L.out_bias, M, d.out_rows, d.out_k, x->y, st);
 }
 
+static RouteArgs routing(const vui_lm_ctx* x, int l, int M) {
+  const vui_lm_layer& L = x->layers[l];
+  RouteArgs r;
+  memset(&r, 0, sizeof(r));
+  r.M = M; r.E = L.experts; r.ldl = x->dims[l].experts16; r.top = L.top; r.tile_rows = moe_tile_rows(x->c.dtype, M, M * L.top, L.experts);
+  r.logits = x->rlog; r.choice = x->choice; r.share = x->share; r.ent = x->ent; r.tile_e = x->tile_e; r.n_tiles = x->n_tiles;
+  return r;
+}
+
 // leaves the outputs in y: one row per position, or per (position, choice) of an expert layer
 static int feed_forward(vui_lm_ctx* x, int l, int M, const LmRows& rows, hipStream_t st) {
   const vui_lm_layer& L = x->layers[l];
@@ -173,11 +182,10 @@ static int feed_forward(vui_lm_ctx* x, int l, int M, const LmRows& rows, hipStre
     return plain(x, d, rows, x->ffa, L.w_down, nullptr, M, d.out_rows, d.ff64, x->y, st);
   }
   if (!lm_rows_routes(M, d.experts16) && (rc = plain(x, d, rows, x->xt, L.w_router, L.router_bias, M, d.experts16, d.w64, x->rlog, st))) return rc;
-  RouteArgs r;
-  memset(&r, 0, sizeof(r));
-  r.M = M; r.E = L.experts; r.ldl = d.experts16; r.top = L.top; r.tile_rows = moe_tile_rows(x->c.dtype, M, M * L.top, L.experts);
-  r.logits = x->rlog; r.choice = x->choice; r.share = x->share; r.ent = x->ent; r.tile_e = x->tile_e; r.n_tiles = x->n_tiles;
-  if ((rc = launch_moe_route(r, st))) return rc;
+  const RouteArgs r = routing(x, l, M);
+  if (!lm_rows_routes(M, d.experts16) || M > 1) {
+    if ((rc = launch_moe_route(r, st))) return rc;
+  }
   up.ent = x->ent; up.tile_e = x->tile_e; up.n_tiles = x->n_tiles; up.top = L.top; up.wz = (size_t)d.ff16 * d.w64;
   up.tile_rows = r.tile_rows;
   up.max_tiles = moe_max_tiles(M * L.top, L.experts, r.tile_rows);
@@ -228,6 +236,7 @@ int sandwich_layers(vui_lm_ctx* x, const int64_t* tokens, int M, const LmRows& r
       RowArgs mid = r;
       if (L.experts > 0 && lm_rows_routes(M, d.experts16)) {
         mid.w_router = L.w_router; mid.router_bias = L.router_bias; mid.experts16 = d.experts16; mid.rlog = x->rlog;
+        mid.route = routing(x, l, M);
       }
       if ((rc = launch_lm_rows(mid, st))) return rc;
       if ((rc = feed_forward(x, l, M, rows, st))) return rc;
