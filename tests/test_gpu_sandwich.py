@@ -75,6 +75,75 @@ def test_prompts_of_many_lengths(name, dt):
         assert e < TOL[dt], (name, T, e)
 
 
+@BOTH
+@pytest.mark.parametrize("name", sorted(SINGLE))
+def test_decoding_of_every_mechanism(name, dt):
+    """Prompts of unequal lengths, then single tokens of all rows together: over tile, block and chunk borders."""
+    cfg = SINGLE[name]()
+    sd = U.sandwich_weights(cfg, 35)
+    eng = U.engine(cfg, sd, dt, max_rows=4, max_seq=160)
+    starts, n = (1, 13, 30, 125), 9
+    seqs = [U.tokens(s + n, cfg["vocab"], s) for s in starts]
+    rows = []
+    for s, toks in zip(starts, seqs):
+        rows.append(eng.new_row())
+        rows[-1].extend(toks[:s])
+    got = []
+    for t in range(n):
+        got.append(eng.decode_step(rows, torch.tensor([toks[s + t] for s, toks in zip(starts, seqs)], device="cuda")).clone())
+    alone = [rows[1].extend([7 % cfg["vocab"]], [0]).clone()]  # and a row by itself
+    for k, (s, toks) in enumerate(zip(starts, seqs)):
+        ref, margins = oracle(cfg, sd, toks + [7 % cfg["vocab"]])
+        mine = torch.stack([g[k] for g in got] + ([alone[0][0]] if k == 1 else []))
+        for j in range(len(mine)):
+            if dt == BF16 and any(m[s + j] < 0.05 for m in margins):
+                continue  # a close call between experts
+            e = U.err(mine[j:j + 1], ref[s + j:s + j + 1])
+            assert e < TOL[dt], (name, s, j, e)
+
+
+@BOTH
+@pytest.mark.parametrize("width,groups", [(80, 16), (84, 4), (30, 3), (66, 1), (1100, 1), (1100, 4), (96, 24), (520, 2), (6, 2)])
+def test_norms_of_many_shapes(width, groups, dt):
+    """Parts that are no whole quads, that several waves share, and more parts than waves, with experts behind them: the
+    router of one row, of few rows and of a prompt."""
+    cfg = U.sandwich([(U.gla(heads=1, dim=4, vdim=4), U.moe(ff=24, experts=7, top=3)), (U.sig(), U.dense(24))], width=width, groups=groups, loop=(1, 2, 2))
+    sd = U.sandwich_weights(cfg, 36)
+    eng = U.engine(cfg, sd, dt, max_seq=120)
+    toks = U.tokens(101, cfg["vocab"], 5)
+    ref, margins = oracle(cfg, sd, toks)
+    with eng.new_row() as row:
+        got = torch.cat([row.extend(toks[:70], range(70)).clone(), row.extend(toks[70:83], range(13)).clone()]
+                        + [row.extend([t], [0]).clone() for t in toks[83:]])
+    e = U.err_clear(got, ref, margins) if dt == BF16 else U.err(got, ref)
+    assert e < TOL[dt], e
+
+
+def test_more_experts_than_the_row_kernel_routes():
+    cfg = U.sandwich([(U.gla(heads=1, dim=4, vdim=4), U.moe(ff=8, experts=200, top=5))])
+    sd = U.sandwich_weights(cfg, 37)
+    eng = U.engine(cfg, sd, F32, max_seq=120)
+    toks = U.tokens(60, cfg["vocab"], 6)
+    ref = O.forward(cfg, sd, toks)
+    with eng.new_row() as row:
+        got = torch.cat([row.extend(toks[:50], range(50)).clone()] + [row.extend([t], [0]).clone() for t in toks[50:]])
+    assert U.err(got, ref) < TOL[F32]
+
+
+@pytest.mark.parametrize("T", [256, 300])
+def test_prompts_on_the_large_tiles(T):
+    """Wide layers and enough positions for tiles of 64 x 64 and 64 x 32, dense and of experts whose rows are put in order."""
+    cfg = U.sandwich([(U.sig(heads=6, kv_heads=3, dim=50, vdim=70), U.dense(2200)), (U.gla(heads=2, dim=90, vdim=150), U.moe(ff=300, experts=5, top=2))],
+                     width=1056, loop=(0, 1, 1))
+    sd = U.sandwich_weights(cfg, 38)
+    eng = U.engine(cfg, sd, BF16, max_seq=320)
+    toks = U.tokens(T, cfg["vocab"], T)
+    ref, margins = oracle(cfg, sd, toks)
+    with eng.new_row() as row:
+        got = run_all(row, toks)
+    assert U.err_clear(got, ref, margins) < TOL[BF16]
+
+
 def test_sizes_of_one():
     cfg = U.sandwich([(U.sig(heads=1, kv_heads=1, dim=1, vdim=1, bias_max=1, buckets=1, q_temp=(0.5, 1)), U.dense(1)),
                       (U.gla(heads=1, dim=1, vdim=1, rank=1), U.moe(ff=1, experts=1, top=1))], width=3, vocab=5, groups=1, eps=1e-2, loop=(0, 1, 1))
