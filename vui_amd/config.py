@@ -322,7 +322,7 @@ class LMConfig:
             layers.append(LMLayerConfig(mixer, mlp))
         out = cls(architecture=arch, width=d["width"], vocab=d["vocab"], norm_eps=d["norm"]["eps"], layers=layers)
         if design.sandwich:
-            out.norm_groups = d["norm"].get("groups") or 1
+            out.norm_groups = d["norm"].get("groups", 1)
             out.embed_scale = (d.get("embedding") or {}).get("scale", 1.0)
             if out.norm_groups < 1 or out.width % out.norm_groups:
                 raise ValueError(f"a width of {out.width} has no {out.norm_groups} equal parts")
